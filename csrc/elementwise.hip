@@ -1,6 +1,6 @@
 // K9/K10/K11 — silu·mul, kv-cache append, residual add.  All HBM-bound:
 // bf16 processed 2..8-wide per thread (G13), grid-stride, capped grids.
-#include "common.h"
+#include "seq_common.h"
 
 namespace {
 
@@ -37,6 +37,21 @@ __global__ void silu_mul2_kernel(const u32* __restrict__ g,
     bf16x2_to_f32(u[idx], u0, u1);
     y[idx] = pack_bf16x2(g0 / (1.f + __expf(-g0)) * u0,
                          g1 / (1.f + __expf(-g1)) * u1);
+  }
+}
+
+// any width, bf16 or fp32 storage
+template <typename T>
+__global__ void silu_mul_any_kernel(const T* __restrict__ gu,
+                                    T* __restrict__ y, u64 rows, int inter) {
+  const u64 total = rows * inter;
+  for (u64 idx = (u64)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+       idx += (u64)gridDim.x * blockDim.x) {
+    const u64 row = idx / inter;
+    const int j = idx % inter;
+    const float g = ldf(gu + row * 2 * inter + j);
+    const float u = ldf(gu + row * 2 * inter + inter + j);
+    stf(y + idx, g / (1.f + expf(-g)) * u);
   }
 }
 
@@ -90,6 +105,20 @@ hipError_t lfmq_silu_mul_fused(const void* gate_up, void* y, long rows,
   u64 total = (u64)rows * (inter / 2);
   hipLaunchKernelGGL(silu_mul_kernel, dim3(grid_for(total)), dim3(256), 0,
                      stream, (const u32*)gate_up, (u32*)y, (u64)rows, inter / 2);
+  return hipGetLastError();
+}
+
+hipError_t lfmq_silu_mul_any(const void* gate_up, void* y, long rows,
+                             int inter, bool f32, hipStream_t stream) {
+  const u64 total = (u64)rows * inter;
+  if (f32)
+    hipLaunchKernelGGL(silu_mul_any_kernel<float>, dim3(grid_for(total)),
+                       dim3(256), 0, stream, (const float*)gate_up, (float*)y,
+                       (u64)rows, inter);
+  else
+    hipLaunchKernelGGL(silu_mul_any_kernel<bf16_t>, dim3(grid_for(total)),
+                       dim3(256), 0, stream, (const bf16_t*)gate_up,
+                       (bf16_t*)y, (u64)rows, inter);
   return hipGetLastError();
 }
 

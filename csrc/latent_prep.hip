@@ -1,0 +1,285 @@
+// Latent attention around the score kernels (attn_window*.hip).
+//
+// latent_prep: one pass over the fused input projection
+//   [ query latent (q_rank) | kv latent (rank) | rotated key (rot) | ... ]
+// norms both latents, rotates the shared key part, and writes the query
+// latent plus the cache row {c [rank], k_rot [rot]} — straight into the
+// ring cache for single-token steps, into the step's key buffer for
+// prompts.
+//
+// The cache keeps the last `cap` tokens of a sequence: position p lives in
+// ring row p mod cap.  latent_ring_load copies the cached tokens that a
+// portion's windows reach back to in front of its own rows;
+// latent_ring_store writes a portion's last `cap` rows back.
+//
+// latent_absorb / latent_expand: small per-head products for decode.  The
+// key up-projection moves to the query (q_abs = q_h W_uk,h, next to the
+// rotated query part) so that scores read the latent cache itself, and the
+// value up-projection to the output, where the partial softmax results of
+// a split key range are merged, the sink joins the denominator and the
+// sigmoid output gate is applied.
+#include "seq_common.h"
+
+namespace {
+
+__device__ __forceinline__ void rope_pair(int pos, float f, float u, float v,
+                                          float& a, float& b) {
+  float s, c;
+  sincosf((float)pos * f, &s, &c);
+  a = u * c - v * s;
+  b = v * c + u * s;
+}
+
+// two waves a row: wave 0 the query latent, wave 1 the cache row
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(
+    const T* __restrict__ in, u64 ld, SeqView sv,
+    const float* __restrict__ wq, const float* __restrict__ wkv,
+    const float* __restrict__ inv_freq, T* __restrict__ cq,
+    T* __restrict__ dst, const i32* __restrict__ dst_row, int cap, int q_rank,
+    int rank, int rot, int rot_dims, float eps) {
+  const int row = blockIdx.x * 2 + (threadIdx.x >> 7);
+  if (row >= sv.n) return;
+  const bool kv = (threadIdx.x >> 6) & 1;
+  const int lane = threadIdx.x & 63;
+  const T* src = in + (u64)row * ld + (kv ? q_rank : 0);
+  const int len = kv ? rank : q_rank;
+  float ss = 0.f;
+  for (int j = lane; j < len; j += 64) {
+    const float a = ldf(src + j);
+    ss = fmaf(a, a, ss);
+  }
+  ss = wave_reduce_sum(ss);
+  const float inv = 1.f / sqrtf(ss / (float)len + eps);
+  if (!kv) {
+    T* o = cq + (u64)row * q_rank;
+    for (int j = lane; j < len; j += 64) stf(o + j, ldf(src + j) * inv * wq[j]);
+    return;
+  }
+  const int s = sv.seq[row];
+  const int slot = sv.slots[s];
+  const int pos = sv.lens[slot] + row - sv.cu[s];
+  const u64 drow = dst_row != nullptr ? (u64)(dst_row[s] + row - sv.cu[s])
+                                      : (u64)slot * cap + pos % cap;
+  T* o = dst + drow * (rank + rot);
+  for (int j = lane; j < len; j += 64) stf(o + j, ldf(src + j) * inv * wkv[j]);
+  const T* kr = src + rank;
+  const int half = rot_dims / 2;
+  for (int j = lane; j < half; j += 64) {
+    float a, b;
+    rope_pair(pos, inv_freq[j], ldf(kr + j), ldf(kr + half + j), a, b);
+    stf(o + rank + j, a);
+    stf(o + rank + half + j, b);
+  }
+  for (int j = rot_dims + lane; j < rot; j += 64) stf(o + rank + j, ldf(kr + j));
+}
+
+// LOAD: key-buffer rows before a sequence's own come from the ring.
+// Otherwise the last min(count, cap) rows of its own go into it.
+template <typename T, bool LOAD>
+__global__ __launch_bounds__(64) void latent_ring_kernel(
+    SeqView sv, const i32* __restrict__ own_row, const i32* __restrict__ prior,
+    T* __restrict__ buf, T* __restrict__ ring, int cap, int d) {
+  const int s = blockIdx.y;
+  const int slot = sv.slots[s];
+  const int len0 = sv.lens[slot], cnt = sv.cu[s + 1] - sv.cu[s];
+  const int total = LOAD ? prior[s] : min(cnt, cap);
+  for (int i = blockIdx.x; i < total; i += gridDim.x) {
+    const int pos = LOAD ? len0 - total + i : len0 + cnt - total + i;
+    T* b = buf + (u64)(own_row[s] + pos - len0) * d;
+    T* r = ring + ((u64)slot * cap + pos % cap) * d;
+    for (int j = threadIdx.x; j < d; j += 64) {
+      if (LOAD) b[j] = r[j]; else r[j] = b[j];
+    }
+  }
+}
+
+constexpr int NB = 8;    // sequences a workgroup serves per weight pass
+
+// y[b, h, n] = sum_k q[b, h, k] W[h, k, n] for n < rank; rotated query
+// part behind it
+template <typename T>
+__global__ __launch_bounds__(256) void latent_absorb_kernel(
+    const T* __restrict__ q, const T* __restrict__ w, SeqView sv,
+    const float* __restrict__ inv_freq, T* __restrict__ out, int heads,
+    int dim, int rot, int rot_dims, int rank) {
+  extern __shared__ float sh[];
+  float* x = sh;                     // [NB][dim]
+  float* red = sh + NB * dim;        // [4][NB][64]
+  const int h = blockIdx.y, b0 = blockIdx.z * NB;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int n = blockIdx.x * 64 + lane;
+  for (int i = threadIdx.x; i < NB * dim; i += 256) {
+    const int bb = b0 + i / dim;
+    x[i] = bb < sv.b
+               ? ldf(q + ((u64)bb * heads + h) * (dim + rot) + i % dim) : 0.f;
+  }
+  __syncthreads();
+  float acc[NB];
+#pragma unroll
+  for (int i = 0; i < NB; ++i) acc[i] = 0.f;
+  if (n < rank) {
+    const T* wp = w + (u64)h * dim * rank + n;
+#pragma unroll 8
+    for (int k = wave; k < dim; k += 4) {
+      const float wv = ldf(wp + (u64)k * rank);
+#pragma unroll
+      for (int i = 0; i < NB; ++i) acc[i] = fmaf(x[i * dim + k], wv, acc[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NB; ++i) red[(wave * NB + i) * 64 + lane] = acc[i];
+  __syncthreads();
+  for (int i = wave; i < NB; i += 4) {
+    const int bb = b0 + i;
+    if (bb >= sv.b) continue;
+    float v = 0.f;
+#pragma unroll
+    for (int g = 0; g < 4; ++g) v += red[(g * NB + i) * 64 + lane];
+    T* o = out + ((u64)bb * heads + h) * (rank + rot);
+    if (n < rank) stf(o + n, v);
+    if (blockIdx.x == 0) {
+      const T* qr = q + ((u64)bb * heads + h) * (dim + rot) + dim;
+      const int pos = sv.lens[sv.slots[bb]];
+      const int half = rot_dims / 2;
+      for (int j = lane; j < half; j += 64) {
+        float a, c;
+        rope_pair(pos, inv_freq[j], ldf(qr + j), ldf(qr + half + j), a, c);
+        stf(o + rank + j, a);
+        stf(o + rank + half + j, c);
+      }
+      for (int j = rot_dims + lane; j < rot; j += 64)
+        stf(o + rank + j, ldf(qr + j));
+    }
+  }
+}
+
+// part [b, splits, heads, rank + 2] = {sum p c, max, sum p} per key range
+template <typename T>
+__global__ __launch_bounds__(256) void latent_expand_kernel(
+    const float* __restrict__ part, int splits, const float* __restrict__ sink,
+    const T* __restrict__ w, const T* __restrict__ g, u64 ldg,
+    T* __restrict__ out, int b, int heads, int rank, int vdim) {
+  extern __shared__ float sh[];
+  float* x = sh;                     // [NB][rank]
+  float* red = sh + NB * rank;       // [4][NB][64]
+  const int h = blockIdx.y, b0 = blockIdx.z * NB;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int n = blockIdx.x * 64 + lane;
+  const u64 pr = rank + 2;
+  for (int i = wave; i < NB; i += 4) {
+    const int bb = b0 + i;
+    if (bb >= b) {
+      for (int j = lane; j < rank; j += 64) x[i * rank + j] = 0.f;
+      continue;
+    }
+    const float* p = part + ((u64)bb * splits * heads + h) * pr;
+    const u64 sp = (u64)heads * pr;
+    float M = sink[h];
+    for (int c = 0; c < splits; ++c) M = fmaxf(M, p[c * sp + rank]);
+    float L = expf(sink[h] - M);
+    for (int c = 0; c < splits; ++c)
+      L += expf(p[c * sp + rank] - M) * p[c * sp + rank + 1];
+    const float inv = 1.f / L;
+    for (int j = lane; j < rank; j += 64) {
+      float a = 0.f;
+      for (int c = 0; c < splits; ++c)
+        a = fmaf(expf(p[c * sp + rank] - M), p[c * sp + j], a);
+      x[i * rank + j] = a * inv;
+    }
+  }
+  __syncthreads();
+  float acc[NB];
+#pragma unroll
+  for (int i = 0; i < NB; ++i) acc[i] = 0.f;
+  if (n < vdim) {
+    const T* wp = w + (u64)h * rank * vdim + n;
+#pragma unroll 8
+    for (int k = wave; k < rank; k += 4) {
+      const float wv = ldf(wp + (u64)k * vdim);
+#pragma unroll
+      for (int i = 0; i < NB; ++i) acc[i] = fmaf(x[i * rank + k], wv, acc[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NB; ++i) red[(wave * NB + i) * 64 + lane] = acc[i];
+  __syncthreads();
+  if (n >= vdim) return;
+  for (int i = wave; i < NB; i += 4) {
+    const int bb = b0 + i;
+    if (bb >= b) continue;
+    float v = 0.f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v += red[(k * NB + i) * 64 + lane];
+    const u64 c = (u64)h * vdim + n;
+    stf(out + (u64)bb * heads * vdim + c,
+        v * sigmoid_f(ldf(g + (u64)bb * ldg + c)));
+  }
+}
+
+}  // namespace
+
+hipError_t lfmq_latent_prep(const void* in, long ld, const SeqView& sv,
+                            const void* wq, const void* wkv,
+                            const void* inv_freq, void* cq, void* dst,
+                            const void* dst_row, int cap, int q_rank,
+                            int rank, int rot, int rot_dims, float eps,
+                            bool f32, hipStream_t stream) {
+  const dim3 grid((sv.n + 1) / 2), block(256);
+#define GO(T)                                                                \
+  hipLaunchKernelGGL(latent_prep_kernel<T>, grid, block, 0, stream,          \
+                     (const T*)in, (u64)ld, sv, (const float*)wq,            \
+                     (const float*)wkv, (const float*)inv_freq, (T*)cq,      \
+                     (T*)dst, (const i32*)dst_row, cap, q_rank, rank, rot,   \
+                     rot_dims, eps)
+  if (f32) GO(float); else GO(bf16_t);
+#undef GO
+  return hipGetLastError();
+}
+
+hipError_t lfmq_latent_ring(const SeqView& sv, const void* own_row,
+                            const void* prior, void* buf, void* ring, int cap,
+                            int d, bool load, bool f32, hipStream_t stream) {
+  const dim3 grid(cap < 256 ? cap : 256, sv.b), block(64);
+#define GO(T, L)                                                             \
+  hipLaunchKernelGGL((latent_ring_kernel<T, L>), grid, block, 0, stream, sv, \
+                     (const i32*)own_row, (const i32*)prior, (T*)buf,        \
+                     (T*)ring, cap, d)
+  if (f32) { if (load) GO(float, true); else GO(float, false); }
+  else { if (load) GO(bf16_t, true); else GO(bf16_t, false); }
+#undef GO
+  return hipGetLastError();
+}
+
+hipError_t lfmq_latent_absorb(const void* q, const void* w, const SeqView& sv,
+                              const void* inv_freq, void* out, int heads,
+                              int dim, int rot, int rot_dims, int rank,
+                              bool f32, hipStream_t stream) {
+  const dim3 grid((rank + 63) / 64, heads, (sv.b + NB - 1) / NB), block(256);
+  const size_t lds = (NB * (size_t)dim + 4 * NB * 64) * sizeof(float);
+  if (lds > 64 * 1024) return hipErrorInvalidValue;
+#define GO(T)                                                                \
+  hipLaunchKernelGGL(latent_absorb_kernel<T>, grid, block, lds, stream,      \
+                     (const T*)q, (const T*)w, sv, (const float*)inv_freq,   \
+                     (T*)out, heads, dim, rot, rot_dims, rank)
+  if (f32) GO(float); else GO(bf16_t);
+#undef GO
+  return hipGetLastError();
+}
+
+hipError_t lfmq_latent_expand(const void* part, int splits, const void* sink,
+                              const void* w, const void* g, long ldg,
+                              void* out, int b, int heads, int rank, int vdim,
+                              bool f32, hipStream_t stream) {
+  const dim3 grid((vdim + 63) / 64, heads, (b + NB - 1) / NB), block(256);
+  const size_t lds = (NB * (size_t)rank + 4 * NB * 64) * sizeof(float);
+  if (lds > 64 * 1024) return hipErrorInvalidValue;
+#define GO(T)                                                                \
+  hipLaunchKernelGGL(latent_expand_kernel<T>, grid, block, lds, stream,      \
+                     (const float*)part, splits, (const float*)sink,         \
+                     (const T*)w, (const T*)g, (u64)ldg, (T*)out, b, heads,  \
+                     rank, vdim)
+  if (f32) GO(float); else GO(bf16_t);
+#undef GO
+  return hipGetLastError();
+}

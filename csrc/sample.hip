@@ -3,7 +3,7 @@
 // reduce has no parallelism there); this two-phase version splits the
 // row over 64 workgroups, then one tiny combine. Ties break to the
 // lowest index (torch semantics).
-#include "common.h"
+#include "seq_common.h"
 
 namespace {
 
@@ -53,6 +53,42 @@ __global__ __launch_bounds__(TPB) void argmax_partial(
   }
 }
 
+// any vocab, bf16 or fp32 logits
+template <typename T>
+__global__ __launch_bounds__(TPB) void argmax_partial_any(
+    const T* __restrict__ logits, float* __restrict__ pmax,
+    i32* __restrict__ pidx, int vocab) {
+  const int row = blockIdx.x, part = blockIdx.y;
+  const int per = (vocab + NSPLIT - 1) / NSPLIT;
+  const int begin = part * per, end = min(begin + per, vocab);
+  const T* src = logits + (u64)row * vocab;
+  float best = -INFINITY;
+  int bidx = begin < vocab ? begin : 0;
+  for (int i = begin + threadIdx.x; i < end; i += TPB) {
+    const float v = ldf(src + i);
+    if (v > best) { best = v; bidx = i; }
+  }
+  __shared__ float smax[TPB / LFMQ_WAVE];
+  __shared__ int sidx[TPB / LFMQ_WAVE];
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const float ob = __shfl_xor(best, off, 64);
+    const int oi = __shfl_xor(bidx, off, 64);
+    if (ob > best || (ob == best && oi < bidx)) { best = ob; bidx = oi; }
+  }
+  const int wave = threadIdx.x / LFMQ_WAVE;
+  if (threadIdx.x % LFMQ_WAVE == 0) { smax[wave] = best; sidx[wave] = bidx; }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int w = 1; w < TPB / LFMQ_WAVE; ++w)
+      if (smax[w] > best || (smax[w] == best && sidx[w] < bidx)) {
+        best = smax[w]; bidx = sidx[w];
+      }
+    pmax[(u64)row * NSPLIT + part] = best;
+    pidx[(u64)row * NSPLIT + part] = bidx;
+  }
+}
+
 __global__ __launch_bounds__(64) void argmax_combine(
     const float* __restrict__ pmax, const i32* __restrict__ pidx,
     long* __restrict__ out) {
@@ -78,6 +114,23 @@ hipError_t lfmq_argmax_rows(const void* logits, void* out, void* scratch_f,
   hipLaunchKernelGGL(argmax_partial, dim3(b, NSPLIT), dim3(TPB), 0, stream,
                      (const u32*)logits, (float*)scratch_f, (i32*)scratch_i,
                      vocab);
+  hipLaunchKernelGGL(argmax_combine, dim3(b), dim3(64), 0, stream,
+                     (const float*)scratch_f, (const i32*)scratch_i,
+                     (long*)out);
+  return hipGetLastError();
+}
+
+hipError_t lfmq_argmax_rows_any(const void* logits, void* out,
+                                void* scratch_f, void* scratch_i, int b,
+                                int vocab, bool f32, hipStream_t stream) {
+  if (f32)
+    hipLaunchKernelGGL(argmax_partial_any<float>, dim3(b, NSPLIT), dim3(TPB),
+                       0, stream, (const float*)logits, (float*)scratch_f,
+                       (i32*)scratch_i, vocab);
+  else
+    hipLaunchKernelGGL(argmax_partial_any<bf16_t>, dim3(b, NSPLIT), dim3(TPB),
+                       0, stream, (const bf16_t*)logits, (float*)scratch_f,
+                       (i32*)scratch_i, vocab);
   hipLaunchKernelGGL(argmax_combine, dim3(b), dim3(64), 0, stream,
                      (const float*)scratch_f, (const i32*)scratch_i,
                      (long*)out);

@@ -7,43 +7,27 @@
 """
 from __future__ import annotations
 
-from typing import Optional, Union
+import os
+from typing import Optional
 
 import torch
 import torch.nn as nn
 
-from .checkpoint import load_meta, load_packed, save_packed
+from .checkpoint import CONFIG_FILE, load_meta, load_packed, save_packed
 from .config import QuantConfig
-from .models.llama import LlamaConfig, LlamaForCausalLM
-from .models.opt import OPTConfig, OPTForCausalLM
 from .models.qlinear import Int8PerTensorLinear, QLinear
+from .models.registry import read_plain_config, spec_of
 from .quant.common import replace_module
 
 
-def build_model(model_cfg: Union[dict, LlamaConfig, OPTConfig], dtype=None,
-                seed: Optional[int] = None) -> nn.Module:
-    """Build a model (random-init if seed given) from a local config."""
+def build_model(model_cfg, dtype=None, seed: Optional[int] = None
+                ) -> nn.Module:
+    """Build a model (random-init if seed given) from a local config (a
+    config object, or a dict naming its arch)."""
+    spec = spec_of(model_cfg)
     if isinstance(model_cfg, dict):
-        arch = model_cfg.get("arch", "llama")
-        if arch == "llama":
-            model_cfg = LlamaConfig.from_dict(model_cfg)
-        elif arch == "opt":
-            model_cfg = OPTConfig.from_dict(model_cfg)
-        elif arch == "mixtral":
-            from .models.mixtral import MixtralConfig
-            model_cfg = MixtralConfig.from_dict(model_cfg)
-        else:
-            raise ValueError(f"unknown arch {arch!r}")
-    arch = model_cfg.arch
-    if arch == "llama":
-        m = LlamaForCausalLM(model_cfg, dtype=dtype or torch.bfloat16)
-    elif arch == "opt":
-        m = OPTForCausalLM(model_cfg, dtype=dtype or torch.float32)
-    elif arch == "mixtral":
-        from .models.mixtral import MixtralForCausalLM
-        m = MixtralForCausalLM(model_cfg, dtype=dtype or torch.bfloat16)
-    else:
-        raise ValueError(f"unknown arch {arch!r}")
+        model_cfg = spec.config.from_dict(model_cfg)
+    m = spec.model(model_cfg, dtype=dtype or spec.dtype)
     if seed is not None:
         m.init_random(seed)
     return m
@@ -55,6 +39,10 @@ def quantize(model: nn.Module, cfg: QuantConfig, calib=None,
     if cfg.fold_rms and getattr(model.cfg, "arch", None) == "llama":
         from .quant.fold import fold_rms_norms
         fold_rms_norms(model)
+    if getattr(model, "packed", False) and cfg.scheme != "rtn":
+        raise NotImplementedError(
+            f"{model.cfg.arch}: per-block calibration ({cfg.scheme}) is not "
+            "implemented, use scheme rtn")
     if cfg.scheme == "rtn":
         from .quant.rtn import RTNQuantizer
         return RTNQuantizer(cfg).run(model)
@@ -111,10 +99,44 @@ def _build_quantized_skeleton(meta: dict, dtype=None) -> nn.Module:
     return model
 
 
+def _fp32_names(model: nn.Module) -> set:
+    """Parameters that stay 32-bit whatever the model's dtype."""
+    fn = getattr(model, "fp32_names", None)
+    return fn() if fn is not None else set()
+
+
+def _load_plain(path: str, plain: dict, device, dtype) -> nn.Module:
+    """config.json + model.safetensors, as trained: one tensor per matrix."""
+    spec = spec_of(plain)
+    cfg = spec.config.from_dict(plain)
+    dtype = dtype or spec.dtype
+    with torch.device("meta"):
+        model = spec.model(cfg, dtype=dtype)
+    keep = _fp32_names(model)
+    state = spec.convert(cfg, load_packed(path))
+    state = {k: v.to(device=device,
+                     dtype=torch.float32 if k in keep else dtype)
+             for k, v in state.items()}
+    for name, p in model.named_parameters():
+        if name in state and state[name].shape != p.shape:
+            raise ValueError(f"{name}: checkpoint has "
+                             f"{tuple(state[name].shape)}, config says "
+                             f"{tuple(p.shape)}")
+    model.load_state_dict(state, strict=True, assign=True)
+    return model
+
+
 def load(path: str, device: str = "cpu", tp_rank: int = 0, tp_world: int = 1,
          dtype=None) -> nn.Module:
-    """Load a packed checkpoint.  tp_world>1: each rank reads only its own
-    shard slices (no broadcast) and gets a TP-sharded module tree."""
+    """Load a packed checkpoint, or a plain one of an architecture that has
+    such a format.  tp_world>1: each rank reads only its own shard slices
+    (no broadcast) and gets a TP-sharded module tree."""
+    if not os.path.exists(os.path.join(path, CONFIG_FILE)):
+        plain = read_plain_config(path)
+        if plain is not None:
+            if tp_world > 1:
+                raise NotImplementedError("plain checkpoints load on one GPU")
+            return _load_plain(path, plain, device, dtype)
     meta = load_meta(path)
     if tp_world > 1:
         from .dist.tp import load_tp
@@ -131,8 +153,9 @@ def load(path: str, device: str = "cpu", tp_rank: int = 0, tp_world: int = 1,
     if dtype is not None:
         # assign=True would otherwise let the checkpoint dtype override an
         # explicitly requested one: cast float tensors here.
-        state = {k: (v.to(dtype) if v.is_floating_point() else v)
-                 for k, v in state.items()}
+        keep = _fp32_names(model)
+        state = {k: (v.to(dtype) if v.is_floating_point() and k not in keep
+                     else v) for k, v in state.items()}
     model.load_state_dict(state, strict=True, assign=True)
     model = model.to(device)  # anything not in the checkpoint (none today)
     # assign=True unties tied embeddings (two independent tensors after the

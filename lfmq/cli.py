@@ -1,15 +1,16 @@
-"""lfmq CLI: quantize / eval / bench / serve.
+"""lfmq CLI: quantize / eval / bench / generate / serve.
 
     python -m lfmq.cli quantize --model llama3-8b --scheme gptq --out ckpt/
     python -m lfmq.cli eval --ckpt ckpt/
     python -m lfmq.cli bench --ckpt ckpt/ --steps 128
+    python -m lfmq.cli generate --ckpt ckpt/ --prompt 1,2,3 --prompt 4,5
     python -m lfmq.cli serve --ckpt ckpt/ --port 8000
 """
 from __future__ import annotations
 
 import json
 import time
-from typing import Optional
+from typing import List, Optional
 
 import torch
 import typer
@@ -24,18 +25,17 @@ MODEL_PRESETS = {
     "tiny-llama": ("llama", "tiny"),
     "tiny-mixtral": ("mixtral", "tiny"),
     "tiny-opt": ("opt", "tiny"),
+    "rapivik-1b": ("rapivik", "sized_1b"),
+    "rapivik-8b": ("rapivik", "sized_8b"),
+    "tiny-rapivik": ("rapivik", "tiny"),
 }
 
 
 def _build_preset(name: str, seed: int, layers: int = 0):
     import lfmq
-    from lfmq.models.llama import LlamaConfig
-    from lfmq.models.mixtral import MixtralConfig
-    from lfmq.models.opt import OPTConfig
+    from lfmq.models.registry import ARCHS
     arch, ctor = MODEL_PRESETS[name]
-    cfg_cls = {"llama": LlamaConfig, "mixtral": MixtralConfig,
-               "opt": OPTConfig}[arch]
-    cfg = getattr(cfg_cls, ctor)()
+    cfg = getattr(ARCHS[arch].config, ctor)()
     if layers:
         cfg.n_layers = layers
     return lfmq.build_model(cfg, seed=seed), cfg
@@ -75,10 +75,14 @@ def quantize(model: str = typer.Option("llama3-8b"),
                             calib_n_seqs=calib_seqs, calib_seq_len=calib_len,
                             act_order=act_order, sym=sym, awq_clip=awq_clip)
     with phase_timer("build model"):
-        m, cfg = _build_preset(model, seed, layers)
-        if hf_dir is not None:
-            from lfmq.models.import_hf import import_hf_state
-            import_hf_state(m, hf_dir)
+        from lfmq.models.registry import read_plain_config
+        if hf_dir is not None and read_plain_config(hf_dir) is not None:
+            m = lfmq.load(hf_dir)       # a registered architecture's own
+        else:
+            m, cfg = _build_preset(model, seed, layers)
+            if hf_dir is not None:
+                from lfmq.models.import_hf import import_hf_state
+                import_hf_state(m, hf_dir)
         m = m.to(dev)
     with phase_timer(f"{scheme} quantize"):
         if scheme == "gptq" and resume:
@@ -97,7 +101,19 @@ def info(ckpt: str = typer.Option(...)):
     """Inspect a packed checkpoint: quant config, model shape, size."""
     import os
 
-    from lfmq.checkpoint import MODEL_FILE, load_meta
+    from lfmq.checkpoint import CONFIG_FILE, MODEL_FILE, load_meta
+    from lfmq.models.registry import read_plain_config, spec_of
+    plain = read_plain_config(ckpt)
+    if plain is not None and not os.path.exists(
+            os.path.join(ckpt, CONFIG_FILE)):
+        cfg = spec_of(plain).config.from_dict(plain)
+        size = os.path.getsize(os.path.join(ckpt, MODEL_FILE))
+        typer.echo(json.dumps({
+            "scheme": None, "arch": cfg.arch, "n_layers": cfg.n_layers,
+            "hidden_size": cfg.hidden_size, "vocab_size": cfg.vocab_size,
+            "file_bytes": size, "file_gib": round(size / (1 << 30), 3),
+        }, indent=2))
+        return
     meta = load_meta(ckpt)
     q = meta["quant"]
     mc = meta["model"]
@@ -206,6 +222,41 @@ def bench(ckpt: Optional[str] = typer.Option(None),
     r = bench_decode(qm, cfg, batch, prompt, steps, warmup, dev,
                      use_graph=not no_graph)
     typer.echo(json.dumps(r, indent=2))
+
+
+@app.command()
+def generate(ckpt: str = typer.Option(...),
+             prompt: List[str] = typer.Option(
+                 ..., help="token ids with commas; repeat for a batch"),
+             max_new_tokens: int = typer.Option(32),
+             dtype: str = typer.Option("", help="bfloat16 | float32; "
+                                       "default: the model's own"),
+             temperature: float = typer.Option(0.0, help="0: greedy"),
+             eos: Optional[int] = typer.Option(None),
+             seed: Optional[int] = typer.Option(None)):
+    """Generate token ids for one or more prompts of token ids.  Prompts
+    of unequal length need a model with packed batches."""
+    import lfmq
+    from lfmq.models.generation import generate_batch
+
+    dev = _device()
+    m = lfmq.load(ckpt, device=dev,
+                  dtype=getattr(torch, dtype) if dtype else None)
+    prompts = [[int(t) for t in p.split(",")] for p in prompt]
+    gc = lfmq.GenerationConfig(max_new_tokens=max_new_tokens,
+                               greedy=temperature <= 0,
+                               temperature=temperature, eos_token_id=eos)
+    gen = None if seed is None else \
+        torch.Generator(device=dev).manual_seed(seed)
+    if getattr(m, "packed", False):
+        out = generate_batch(m, prompts, gen_cfg=gc, generator=gen)
+    else:
+        if len(set(map(len, prompts))) > 1:
+            raise typer.BadParameter("this model takes prompts of one length")
+        out = m.generate(torch.tensor(prompts, device=dev), gen_cfg=gc,
+                         generator=gen).tolist()
+    for row in out:
+        typer.echo(",".join(map(str, row)))
 
 
 @app.command()

@@ -12,12 +12,12 @@ end.  torch.cuda.CUDAGraph is hipGraph on ROCm.
 """
 from __future__ import annotations
 
-from typing import Optional
+from typing import Optional, Sequence
 
 import torch
 
 from ..ops import functional as F
-from ..ops import hip_ext
+from ..ops import seq_ext
 
 
 class GraphDecoder:
@@ -40,8 +40,8 @@ class GraphDecoder:
     def _step(self):
         logits = self.model.forward_decode_step(
             self.tok.unsqueeze(1), self.cache, self.state, self.max_seq)
-        sampled = hip_ext().greedy_sample(logits[:, -1].contiguous())
-        hip_ext().advance_record(self.state, self.tok, sampled, self.ring)
+        sampled = F.greedy_sample(logits[:, -1])
+        seq_ext().advance_record(self.state, self.tok, sampled, self.ring)
 
     @torch.no_grad()
     def capture(self):
@@ -58,12 +58,15 @@ class GraphDecoder:
             self._step()
 
     @torch.no_grad()
-    def prefill(self, input_ids: torch.Tensor) -> None:
-        """Eager prefill + set up the device state for decode."""
+    def prefill(self, input_ids: torch.Tensor,
+                lengths: Optional[Sequence[int]] = None) -> None:
+        """Eager prefill + set up the device state for decode.  lengths:
+        row i holds lengths[i] tokens (models with packed batches)."""
         b, L = input_ids.shape
         assert b == self.batch
         self.cache.reset()
-        logits = self.model(input_ids.to(self.device), self.cache)
+        kw = {} if lengths is None else {"lengths": lengths}
+        logits = self.model(input_ids.to(self.device), self.cache, **kw)
         first = F.greedy_sample(logits[:, -1].contiguous())
         self.tok.copy_(first)
         self.state.copy_(torch.tensor([L, L + 1, 0], dtype=torch.int32))
@@ -88,16 +91,17 @@ class GraphDecoder:
         if self.graph is None:
             # capture AFTER a real prefill so shapes/addresses are final
             saved = (self.state.clone(), self.tok.clone(),
-                     self.cache.seq_len)
+                     self.cache.snapshot())
             self.capture()
             self.state.copy_(saved[0])
             self.tok.copy_(saved[1])
-            self.cache.seq_len = saved[2]
+            self.cache.restore(saved[2])
+            self.ring.zero_()
         start = self.step_count
         for _ in range(n_tokens):
             self.graph.replay()
         self.step_count += n_tokens
-        self.cache.seq_len += n_tokens
+        self.cache.replayed(n_tokens)
         eng = getattr(self.model, "_engine", None)
         if eng is not None:
             eng.check_health()  # surfaces engine spin give-up codes

@@ -30,3 +30,15 @@ class KVCache:
         self.seq_len += n
         if self.seq_len > self.max_seq:
             raise RuntimeError(f"KV cache overflow: {self.seq_len} > {self.max_seq}")
+
+    def replayed(self, n: int) -> None:
+        """n captured decode steps ran on the device."""
+        self.seq_len += n
+
+    def snapshot(self):
+        """What a warm-up step would change: rows past seq_len are written
+        again by the step that owns them, so the length is all of it."""
+        return self.seq_len
+
+    def restore(self, snap) -> None:
+        self.seq_len = snap

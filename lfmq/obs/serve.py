@@ -19,7 +19,7 @@ import time
 from typing import Dict, List
 
 import torch
-from fastapi import FastAPI
+from fastapi import FastAPI, HTTPException
 from pydantic import BaseModel
 from prometheus_client import (CONTENT_TYPE_LATEST, Counter, Gauge,
                                generate_latest)
@@ -45,6 +45,22 @@ def make_app(model) -> FastAPI:
     graph_decoders: Dict[int, object] = {}   # batch size -> GraphDecoder
     graph_lock = threading.Lock()
 
+    def _generate_unequal(req: GenRequest, gc, gen):
+        """Prompts of unequal length: packed-batch models only."""
+        if not getattr(model, "packed", False):
+            raise HTTPException(400, "this model takes prompts of one length")
+        from ..models.generation import generate_batch
+        t0 = time.perf_counter()
+        with graph_lock:
+            out = generate_batch(model, req.input_ids, gen_cfg=gc,
+                                 generator=gen)
+        dt = time.perf_counter() - t0
+        new = sum(map(len, out)) - sum(map(len, req.input_ids))
+        TOKS.inc(new)
+        TOKS_PER_S.set(new / max(dt, 1e-9))
+        return {"output_ids": out, "seconds": dt, "new_tokens":
+                max(len(o) - len(p) for o, p in zip(out, req.input_ids))}
+
     def _graph_generate(ids: torch.Tensor, max_new: int) -> torch.Tensor:
         from ..models.graph import GraphDecoder
         b = ids.shape[0]
@@ -68,8 +84,12 @@ def make_app(model) -> FastAPI:
     @app.post("/generate")
     def generate(req: GenRequest):
         REQS.inc()
-        ids = torch.tensor(req.input_ids, dtype=torch.int64, device=device)
         from ..config import GenerationConfig
+        vocab = model.cfg.vocab_size
+        if not req.input_ids or not all(req.input_ids) or not all(
+                0 <= t < vocab for p in req.input_ids for t in p):
+            raise HTTPException(400, "input_ids must be non-empty lists of "
+                                     f"token ids below {vocab}")
         gc = GenerationConfig(max_new_tokens=req.max_new_tokens,
                               greedy=req.greedy, temperature=req.temperature,
                               eos_token_id=req.eos_token_id)
@@ -77,6 +97,9 @@ def make_app(model) -> FastAPI:
         if req.seed is not None:
             # generator device must match the logits device (multinomial)
             gen = torch.Generator(device=str(device)).manual_seed(req.seed)
+        if len(set(map(len, req.input_ids))) > 1:
+            return _generate_unequal(req, gc, gen)
+        ids = torch.tensor(req.input_ids, dtype=torch.int64, device=device)
         t0 = time.perf_counter()
         use_graph = (device.type == "cuda" and req.greedy
                      and req.max_new_tokens > 0)

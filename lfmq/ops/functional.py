@@ -14,7 +14,7 @@ from typing import Optional
 
 import torch
 
-from . import hip_ext, ref
+from . import hip_ext, ref, seq_ext
 
 # Debug numeric guard: LFMQ_NANCHECK=1 asserts every op
 # output is finite — catches kernel-layout or quantization bugs at the
@@ -108,7 +108,7 @@ def silu_mul_gateup(gate_up: torch.Tensor, inter: int) -> torch.Tensor:
     """silu(gu[..., :inter]) * gu[..., inter:] without materializing the
     split halves (one fused kernel on GPU)."""
     if gate_up.is_cuda:
-        return hip_ext().silu_mul_fused(gate_up.contiguous())
+        return seq_ext().silu_mul_fused(gate_up.contiguous())
     gate, up = gate_up.split([inter, inter], dim=-1)
     return ref.silu_mul(gate, up)
 
@@ -237,7 +237,7 @@ def dq_gemv_gateup(x: torch.Tensor, qweight: torch.Tensor,
 def greedy_sample(logits: torch.Tensor) -> torch.Tensor:
     """argmax over the last dim of [b, vocab] logits -> int64 [b]."""
     if logits.is_cuda:
-        return hip_ext().greedy_sample(logits.contiguous())
+        return seq_ext().greedy_sample(logits.contiguous())
     return logits.argmax(dim=-1)
 
 
@@ -249,3 +249,93 @@ def kv_append(k_cache, v_cache, k_new, v_new, pos: int) -> None:
                             v_new.contiguous(), pos)
         return
     ref.kv_append(k_cache, v_cache, k_new.transpose(1, 2), v_new.transpose(1, 2), pos)
+
+
+# ---------------------------------------------------------------------------
+# packed-batch ops (lfmq/models/seqcache.py: StepBatch).  GPU only.
+# ---------------------------------------------------------------------------
+
+def bigram_embed(tokens, batch, cache, embed, table, mul_prev: int,
+                 mul_cur: int) -> torch.Tensor:
+    """fp32 residual rows embed[tok] + table[hash(prev, tok)]; a sequence's
+    first token takes the table's last row."""
+    return seq_ext().bigram_embed(tokens, *batch.view(cache), cache.prev,
+                                  embed, table, mul_prev, mul_cur)
+
+
+def seq_advance(tokens, batch, cache) -> None:
+    """Close a step on the device: lengths, previous tokens, buffer turns."""
+    seq_ext().seq_advance(tokens, batch.cu, batch.slots, cache.lens,
+                          cache.prev, cache.turn)
+
+
+def add_norm(x, y, weight, bias: float, eps: float, out_dtype,
+             side_w=None, side_b=None):
+    """x += y in place (fp32 residual), then h = rms_norm(x) * (bias + w).
+    Returns (h, side): side = h @ side_w^T + side_b in fp32."""
+    h, side = seq_ext().add_norm(x, y, weight, bias, eps, side_w, side_b,
+                                 out_dtype == torch.float32)
+    return _guard(h, "add_norm"), side
+
+
+def mlstm(qkv, gates, batch, cache, S, nm, cap: float) -> torch.Tensor:
+    """Matrix-memory recurrence over the step's rows: fp32 [N, H, vdim]."""
+    return _guard(seq_ext().mlstm_scan(qkv, gates, *batch.view(cache),
+                                       cache.turn, S, nm, cap), "mlstm")
+
+
+def head_norm_gate(o, gate, weight, eps: float) -> torch.Tensor:
+    return _guard(seq_ext().head_norm_gate(o, gate, weight, eps),
+                  "head_norm_gate")
+
+
+def rope_inv_freq(dims: int, base: float, device) -> torch.Tensor:
+    """fp32 base^(-2i/dims), i < dims/2, from a double-precision power."""
+    key = ("f64", dims, float(base), str(device))
+    t = _INV_FREQ_CACHE.get(key)
+    if t is None:
+        i = torch.arange(dims // 2, dtype=torch.float64)
+        t = (float(base) ** (-2.0 * i / dims)).float().to(device)
+        _INV_FREQ_CACHE[key] = t
+    return t
+
+
+def latent_prep(proj, batch, cache, q_norm, kv_norm, inv_freq, dst, dst_row,
+                eps: float) -> torch.Tensor:
+    return seq_ext().latent_prep(proj, *batch.view(cache), q_norm, kv_norm,
+                                 inv_freq, dst, dst_row, eps)
+
+
+def latent_ring(batch, cache, rows, buf, ring, load: bool) -> None:
+    seq_ext().latent_ring(*batch.view(cache), rows.own, rows.prior, buf, ring,
+                          load)
+
+
+def latent_absorb(q, w_uk, batch, cache, inv_freq, rot: int) -> torch.Tensor:
+    return seq_ext().latent_absorb(q, w_uk, *batch.view(cache), inv_freq, rot)
+
+
+def latent_expand(part, sink, w_uv, gate) -> torch.Tensor:
+    return _guard(seq_ext().latent_expand(part, sink, w_uv, gate),
+                  "latent_expand")
+
+
+def attn_window_prompt(q, kv, lat, batch, cache, rows, inv_freq, sink, gate,
+                       d1: int, d2: int, dv: int, window: int,
+                       scale: float) -> torch.Tensor:
+    """Sliding-window attention with a sink and an output gate over the
+    step's key buffer (q's second part is rotated inside)."""
+    return _guard(seq_ext().attn_window_prompt(
+        q, kv, lat, *batch.view(cache), rows.own, inv_freq, sink, gate, d1,
+        d2, dv, window, scale), "attn_window_prompt")
+
+
+def attn_window_decode(q, ring, batch, cache, rank: int, window: int,
+                       scale: float) -> torch.Tensor:
+    """Absorbed queries over the latent ring: partial results of a split
+    key range (one token per sequence)."""
+    reach = min(window, ring.shape[1])
+    # enough key ranges to fill the chip, none shorter than a key tile
+    splits = max(1, min(-(-reach // 64), -(-1024 // (q.shape[0] * q.shape[1]))))
+    return seq_ext().attn_window_decode(q, ring, *batch.view(cache), rank,
+                                        window, splits, scale)

@@ -1,9 +1,13 @@
-"""In-tree build of the lfmq_hip extension (gfx950 only).
+"""In-tree build of the gfx950 HIP extensions.
 
     PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace
 
-The built lfmq_hip*.so lands at the repo root so it travels with gpurun
-snapshots (a JIT cache under ~/.cache would not).
+  lfmq_hip  weight-quantized Llama / Mixtral / OPT kernels
+  lfmq_seq  recurrent and latent-attention layers, packed batches, and the
+            small ops that every model uses
+
+LFMQ_EXTENSIONS=lfmq_seq builds only the named ones (comma-separated).
+The built .so files land at the repo root, next to the package.
 """
 import os
 
@@ -39,17 +43,37 @@ SOURCES = [
     "csrc/moe_route.hip",
 ]
 
+SEQ_SOURCES = [
+    "csrc/seq_ext.hip",
+    "csrc/bigram_embed.hip",
+    "csrc/fused_norm.hip",
+    "csrc/mlstm.hip",
+    "csrc/latent_prep.hip",
+    "csrc/attn_window.hip",
+    "csrc/elementwise.hip",
+    "csrc/sample.hip",
+]
+
+# packed fp32 instructions off: some of their forms have returned wrong
+# results on this hardware
+_HIP_FLAGS = ["-O3", "-std=c++17", "-Xclang", "-target-feature",
+              "-Xclang", "-packed-fp32-ops"]
+
+_ALL = {"lfmq_hip": SOURCES, "lfmq_seq": SEQ_SOURCES}
+_WANT = [n for n in os.environ.get("LFMQ_EXTENSIONS", "").split(",") if n]
+for _n in _WANT:
+    if _n not in _ALL:
+        raise SystemExit(f"LFMQ_EXTENSIONS: unknown extension {_n!r}")
+
 setup(
     name="lfmq_hip",
     ext_modules=[
         CUDAExtension(
-            name="lfmq_hip",
-            sources=SOURCES,
-            extra_compile_args={
-                "cxx": _CXX_FLAGS,
-                "nvcc": ["-O3", "-std=c++17"],
-            },
+            name=name,
+            sources=sources,
+            extra_compile_args={"cxx": _CXX_FLAGS, "nvcc": _HIP_FLAGS},
         )
+        for name, sources in _ALL.items() if not _WANT or name in _WANT
     ],
     cmdclass={"build_ext": BuildExtension.with_options(use_ninja=True)},
 )
