@@ -25,6 +25,11 @@ hipError_t lfmq_head_norm_gate(const void*, const void*, long, const void*,
 hipError_t lfmq_mlstm_scan(const void*, long, const void*, const SeqView&,
                            const void*, void*, void*, void*, int, int, int,
                            float, bool, hipStream_t);
+bool lfmq_mlstm_chunk_ok(const void*, long, int, int);
+hipError_t lfmq_mlstm_chunk(const void*, long, const void*, const SeqView&,
+                            const void*, const void*, void*, void*, void*,
+                            void*, void*, const void*, void*, int, int, int,
+                            float, float, int, int, hipStream_t);
 hipError_t lfmq_latent_prep(const void*, long, const SeqView&, const void*,
                             const void*, const void*, void*, void*,
                             const void*, int, int, int, int, int, float, bool,
@@ -46,6 +51,13 @@ hipError_t lfmq_attn_window_prompt(const void*, const void*, long, long,
 hipError_t lfmq_attn_window_decode(const void*, const void*, const SeqView&,
                                    void*, int, int, int, int, int, int, float,
                                    bool, hipStream_t);
+bool lfmq_attn_window_prompt_mfma_ok(const void*, const void*, long,
+                                     const void*, long, const void*, long, int,
+                                     int, int);
+hipError_t lfmq_attn_window_prompt_mfma(
+    const void*, const void*, long, const void*, long, const void*, long,
+    const SeqView&, const void*, const void*, const void*, const void*, long,
+    void*, int, int, int, int, int, int, float, int, hipStream_t);
 hipError_t lfmq_silu_mul_fused(const void*, void*, long, int, hipStream_t);
 hipError_t lfmq_silu_mul_any(const void*, void*, long, int, bool,
                              hipStream_t);
@@ -219,6 +231,44 @@ T_ mlstm_scan(T_ qkv, T_ gates, T_ seq, T_ cu, T_ slots, T_ lens, T_ turn,
   return out;
 }
 
+// whether the chunk kernels take this projection's shape
+bool mlstm_chunk_ok(T_ qkv, T_ S) {
+  return qkv.scalar_type() == torch::kBFloat16 && qkv.dim() == 2 &&
+         qkv.stride(1) == 1 &&
+         lfmq_mlstm_chunk_ok(qkv.data_ptr(), qkv.stride(0), (int)S.size(2),
+                             (int)S.size(3));
+}
+
+// qkv rows [q | k | v | gate]; chunk_base [b] first chunk of each sequence,
+// `chunks` in all, L tokens each.  Returns the normed and gated [N, H vdim].
+T_ mlstm_chunk(T_ qkv, T_ gates, T_ seq, T_ cu, T_ slots, T_ lens, T_ turn,
+               T_ S, T_ nm, double cap, T_ norm_w, double eps, T_ chunk_base,
+               long chunks, long L, long max_count) {
+  const SeqView sv = view(seq, cu, slots, lens);
+  check_mlstm(qkv, gates, sv, lens, turn, S, nm);
+  check(norm_w, torch::kFloat32, "norm weight");
+  check(chunk_base, torch::kInt32, "chunk_base");
+  const long H = S.size(1), dim = S.size(2), V = S.size(3);
+  TORCH_CHECK(mlstm_chunk_ok(qkv, S), "mlstm_chunk: shape not supported");
+  const long ld = row_stride(qkv, 2 * H * (dim + V), "qkv");
+  TORCH_CHECK(norm_w.numel() == H * V && chunk_base.numel() == sv.b &&
+                  chunks >= sv.b && max_count >= 1,
+              "mlstm_chunk: shape mismatch");
+  const long DP = (dim + 63) / 64 * 64, VP = (V + 63) / 64 * 64;
+  auto f = S.options();
+  auto ws = torch::empty({chunks * H * 2 * VP * DP}, qkv.options());
+  auto nws = torch::empty({chunks * H * DP}, f);
+  auto gws = torch::empty({3 * H * sv.n}, f);
+  auto out = torch::empty({sv.n, H * V}, qkv.options());
+  CHECK_HIP(lfmq_mlstm_chunk(
+      qkv.data_ptr(), ld, gates.data_ptr(), sv, turn.data_ptr(),
+      chunk_base.data_ptr(), S.data_ptr(), nm.data_ptr(), ws.data_ptr(),
+      nws.data_ptr(), gws.data_ptr(), norm_w.data_ptr(), out.data_ptr(),
+      (int)H, (int)dim, (int)V, (float)cap, (float)eps, (int)L,
+      (int)max_count, stream()));
+  return out;
+}
+
 // dst_row given: rows of `dst` [rows, rank + rot]; else dst is the ring
 // [slots, cap, rank + rot].  Returns the normed query latent.
 T_ latent_prep(T_ in, T_ seq, T_ cu, T_ slots, T_ lens, T_ wq, T_ wkv,
@@ -321,7 +371,8 @@ T_ latent_expand(T_ part, T_ sink, T_ w, T_ g) {
 // values; lat [rows, rank + d2] whose tail is the shared key part
 T_ attn_window_prompt(T_ q, T_ kv, T_ lat, T_ seq, T_ cu, T_ slots, T_ lens,
                       T_ own_row, T_ inv_freq, T_ sink, T_ g, long d1, long d2,
-                      long dv, long window, double scale) {
+                      long dv, long window, double scale, long max_count,
+                      bool general) {
   const SeqView sv = view(seq, cu, slots, lens);
   const bool f32 = storage(q, "q");
   const auto dt = q.scalar_type();
@@ -342,10 +393,21 @@ T_ attn_window_prompt(T_ q, T_ kv, T_ lat, T_ seq, T_ cu, T_ slots, T_ lens,
   auto out = torch::empty({sv.n, H * dv}, q.options());
   const long ld = kv.size(1), ll = lat.size(1);
   const size_t es = q.element_size();
+  const void* k2 = (const char*)lat.data_ptr() + (ll - d2) * es;
+  const void* vp = (const char*)kv.data_ptr() + H * d1 * es;
+  if (!f32 && !general &&
+      lfmq_attn_window_prompt_mfma_ok(q.data_ptr(), kv.data_ptr(), ld, k2, ll,
+                                      vp, ld, (int)d1, (int)d2, (int)dv)) {
+    CHECK_HIP(lfmq_attn_window_prompt_mfma(
+        q.data_ptr(), kv.data_ptr(), ld, k2, ll, vp, ld, sv,
+        own_row.data_ptr(), inv_freq.data_ptr(), sink.data_ptr(),
+        g.data_ptr(), ldg, out.data_ptr(), (int)H, (int)d1, (int)d2,
+        (int)(2 * inv_freq.numel()), (int)dv, (int)window, (float)scale,
+        (int)max_count, stream()));
+    return out;
+  }
   CHECK_HIP(lfmq_attn_window_prompt(
-      q.data_ptr(), kv.data_ptr(), ld, d1,
-      (const char*)lat.data_ptr() + (ll - d2) * es, ll,
-      (const char*)kv.data_ptr() + H * d1 * es, ld, dv, sv,
+      q.data_ptr(), kv.data_ptr(), ld, d1, k2, ll, vp, ld, dv, sv,
       own_row.data_ptr(), inv_freq.data_ptr(), sink.data_ptr(), g.data_ptr(),
       ldg, out.data_ptr(), (int)H, (int)d1, (int)d2,
       (int)(2 * inv_freq.numel()), (int)dv, (int)window, (float)scale, f32,
@@ -428,6 +490,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("add_norm", &add_norm, "fp32 residual add + norm + side projection");
   m.def("head_norm_gate", &head_norm_gate, "per-head norm, weight and gate");
   m.def("mlstm_scan", &mlstm_scan, "matrix-memory recurrence, token by token");
+  m.def("mlstm_chunk_ok", &mlstm_chunk_ok, "shape check of mlstm_chunk");
+  m.def("mlstm_chunk", &mlstm_chunk,
+        "matrix-memory recurrence by chunks, normed and gated");
   m.def("latent_prep", &latent_prep, "latent norms + shared rotated key");
   m.def("latent_ring", &latent_ring, "ring cache <-> step key buffer");
   m.def("latent_absorb", &latent_absorb, "queries into the latent space");

@@ -67,9 +67,9 @@ class MLSTMMixer(nn.Module):
 
     def forward(self, h, side, batch, cache, state):
         p = self.in_proj(h)
-        o = F.mlstm(p, side, batch, cache, state["S"], state["nm"], self.cap)
-        gate = p[:, self.heads * (2 * self.dim + self.vdim):]
-        return self.o_proj(F.head_norm_gate(o, gate, self.norm_w, self.eps))
+        return self.o_proj(F.mlstm(p, side, batch, cache, state["S"],
+                                   state["nm"], self.cap, self.norm_w,
+                                   self.eps))
 
 
 class LatentAttention(nn.Module):

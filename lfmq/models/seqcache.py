@@ -46,6 +46,7 @@ class StepBatch:
         self.cu = t[self.n:self.n + self.b + 1]
         self.slots = t[self.n + self.b + 1:]
         self._rows: Dict[int, SimpleNamespace] = {}
+        self._chunks: Dict[int, tuple] = {}
 
     def _dev(self, ints) -> torch.Tensor:
         return torch.tensor(ints, dtype=torch.int32).to(self.device)
@@ -70,6 +71,18 @@ class StepBatch:
                                 any_prior=any(prior))
             self._rows[window] = r
         return r
+
+
+    def chunks(self, size: int):
+        """(first chunk of every sequence, chunks in all) when sequences
+        are cut into chunks of `size` tokens."""
+        if size not in self._chunks:
+            base, at = [], 0
+            for c in self.counts:
+                base.append(at)
+                at += -(-c // size)
+            self._chunks[size] = (self._dev(base), at)
+        return self._chunks[size]
 
 
 class SequenceCache:

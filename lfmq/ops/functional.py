@@ -278,13 +278,28 @@ def add_norm(x, y, weight, bias: float, eps: float, out_dtype,
     return _guard(h, "add_norm"), side
 
 
-def mlstm(qkv, gates, batch, cache, S, nm, cap: float) -> torch.Tensor:
-    """Matrix-memory recurrence over the step's rows: fp32 [N, H, vdim]."""
-    return _guard(seq_ext().mlstm_scan(qkv, gates, *batch.view(cache),
-                                       cache.turn, S, nm, cap), "mlstm")
+MLSTM_CHUNK = 128        # tokens a chunk: state traffic against score work
+
+
+def mlstm(proj, gates, batch, cache, S, nm, cap: float, norm_w, eps: float,
+          by_token: bool = False) -> torch.Tensor:
+    """Matrix-memory recurrence over the step's rows, each head's output
+    normed, weighted and gated: [N, H * vdim].  proj rows are
+    [q | k | v | output gate].  Single tokens and 32-bit storage run token
+    by token (by_token: everything), prompts by chunks."""
+    ext = seq_ext()
+    if not (by_token or batch.single) and ext.mlstm_chunk_ok(proj, S):
+        base, total = batch.chunks(MLSTM_CHUNK)
+        return _guard(ext.mlstm_chunk(
+            proj, gates, *batch.view(cache), cache.turn, S, nm, cap, norm_w,
+            eps, base, total, MLSTM_CHUNK, max(batch.counts)), "mlstm_chunk")
+    o = ext.mlstm_scan(proj, gates, *batch.view(cache), cache.turn, S, nm, cap)
+    gate = proj[:, S.shape[1] * (2 * S.shape[2] + S.shape[3]):]
+    return head_norm_gate(o, gate, norm_w, eps)
 
 
 def head_norm_gate(o, gate, weight, eps: float) -> torch.Tensor:
+    """o / rms(o) per head (fp32 [N, H, v]), times weight and sigmoid(gate)."""
     return _guard(seq_ext().head_norm_gate(o, gate, weight, eps),
                   "head_norm_gate")
 
@@ -321,13 +336,15 @@ def latent_expand(part, sink, w_uv, gate) -> torch.Tensor:
 
 
 def attn_window_prompt(q, kv, lat, batch, cache, rows, inv_freq, sink, gate,
-                       d1: int, d2: int, dv: int, window: int,
-                       scale: float) -> torch.Tensor:
+                       d1: int, d2: int, dv: int, window: int, scale: float,
+                       general: bool = False) -> torch.Tensor:
     """Sliding-window attention with a sink and an output gate over the
-    step's key buffer (q's second part is rotated inside)."""
+    step's key buffer (q's second part is rotated inside).  general: the
+    any-size kernel also where the matrix-core one applies."""
     return _guard(seq_ext().attn_window_prompt(
         q, kv, lat, *batch.view(cache), rows.own, inv_freq, sink, gate, d1,
-        d2, dv, window, scale), "attn_window_prompt")
+        d2, dv, window, scale, max(batch.counts), general),
+        "attn_window_prompt")
 
 
 def attn_window_decode(q, ring, batch, cache, rank: int, window: int,

@@ -48,8 +48,10 @@ SEQ_SOURCES = [
     "csrc/bigram_embed.hip",
     "csrc/fused_norm.hip",
     "csrc/mlstm.hip",
+    "csrc/mlstm_chunk.hip",
     "csrc/latent_prep.hip",
     "csrc/attn_window.hip",
+    "csrc/attn_window_mfma.hip",
     "csrc/elementwise.hip",
     "csrc/sample.hip",
 ]
