@@ -41,9 +41,29 @@ def main():
                     help="legacy alias for --lm-head w4")
     ap.add_argument("--no-fidelity", action="store_true",
                     help="skip the delta-ppl/logit-KL fidelity pass")
+    ap.add_argument("--compare", default="", metavar="SIZE",
+                    help="instead: prefill and decode throughput of Rapivik "
+                         "beside Llama at equal sizes (2k, 4k), one JSON "
+                         "line per shape")
+    ap.add_argument("--phase", default="", choices=["", "prefill", "decode"],
+                    help="with --compare: only this phase")
+    ap.add_argument("--shape", default="", metavar="BATCHxLENGTH",
+                    help="with --compare: only this shape")
     args = ap.parse_args()
 
     sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
+    if args.compare:
+        from lfmq.bench.compare import DECODE, PREFILL, compare
+        pre, dec = PREFILL, DECODE
+        if args.shape:
+            b, n = map(int, args.shape.split("x"))
+            pre = dec = ((b, n),)
+        for row in compare(args.compare, args.layers or 8,
+                           prefill=() if args.phase == "decode" else pre,
+                           decode=() if args.phase == "prefill" else dec):
+            print(json.dumps(row), flush=True)
+        return
+
     import lfmq.dist as lfmq_dist
     from lfmq.bench.decode import bench_decode, build_quantized_llama
 

@@ -94,50 +94,65 @@ __global__ __launch_bounds__(64) void latent_ring_kernel(
   }
 }
 
-constexpr int NB = 8;    // sequences a workgroup serves per weight pass
+constexpr int PTPB = 512, PW = PTPB / 64;   // per-head products
 
-// y[b, h, n] = sum_k q[b, h, k] W[h, k, n] for n < rank; rotated query
-// part behind it
-template <typename T>
-__global__ __launch_bounds__(256) void latent_absorb_kernel(
-    const T* __restrict__ q, const T* __restrict__ w, SeqView sv,
-    const float* __restrict__ inv_freq, T* __restrict__ out, int heads,
-    int dim, int rot, int rot_dims, int rank) {
-  extern __shared__ float sh[];
-  float* x = sh;                     // [NB][dim]
-  float* red = sh + NB * dim;        // [4][NB][64]
-  const int h = blockIdx.y, b0 = blockIdx.z * NB;
+// acc[i] = sum_k x[i][k] w[k][col] over this wave's share of k, then over
+// the waves through red [PW][NB][64]
+template <typename T, int NB>
+__device__ __forceinline__ void head_product(const float* x, int kdim,
+                                             const T* w, int ncol, int n,
+                                             float* red) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int n = blockIdx.x * 64 + lane;
-  for (int i = threadIdx.x; i < NB * dim; i += 256) {
-    const int bb = b0 + i / dim;
-    x[i] = bb < sv.b
-               ? ldf(q + ((u64)bb * heads + h) * (dim + rot) + i % dim) : 0.f;
-  }
-  __syncthreads();
   float acc[NB];
 #pragma unroll
   for (int i = 0; i < NB; ++i) acc[i] = 0.f;
-  if (n < rank) {
-    const T* wp = w + (u64)h * dim * rank + n;
-#pragma unroll 8
-    for (int k = wave; k < dim; k += 4) {
-      const float wv = ldf(wp + (u64)k * rank);
+  if (n < ncol) {
+    const T* wp = w + n;
+#pragma unroll 16
+    for (int k = wave; k < kdim; k += PW) {
+      const float wv = ldf(wp + (u64)k * ncol);
 #pragma unroll
-      for (int i = 0; i < NB; ++i) acc[i] = fmaf(x[i * dim + k], wv, acc[i]);
+      for (int i = 0; i < NB; ++i) acc[i] = fmaf(x[i * kdim + k], wv, acc[i]);
     }
   }
 #pragma unroll
   for (int i = 0; i < NB; ++i) red[(wave * NB + i) * 64 + lane] = acc[i];
   __syncthreads();
-  for (int i = wave; i < NB; i += 4) {
+}
+
+template <int NB>
+__device__ __forceinline__ float head_sum(const float* red, int i, int lane) {
+  float v = 0.f;
+#pragma unroll
+  for (int g = 0; g < PW; ++g) v += red[(g * NB + i) * 64 + lane];
+  return v;
+}
+
+// y[b, h, n] = sum_k q[b, h, k] W[h, k, n] for n < rank; rotated query
+// part behind it.  NB sequences share a pass over the weights.
+template <typename T, int NB>
+__global__ __launch_bounds__(PTPB) void latent_absorb_kernel(
+    const T* __restrict__ q, const T* __restrict__ w, SeqView sv,
+    const float* __restrict__ inv_freq, T* __restrict__ out, int heads,
+    int dim, int rot, int rot_dims, int rank) {
+  extern __shared__ float sh[];
+  float* x = sh;                     // [NB][dim]
+  float* red = sh + NB * dim;        // [PW][NB][64]
+  const int h = blockIdx.y, b0 = blockIdx.z * NB;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int n = blockIdx.x * 64 + lane;
+  for (int i = threadIdx.x; i < NB * dim; i += PTPB) {
+    const int bb = b0 + i / dim;
+    x[i] = bb < sv.b
+               ? ldf(q + ((u64)bb * heads + h) * (dim + rot) + i % dim) : 0.f;
+  }
+  __syncthreads();
+  head_product<T, NB>(x, dim, w + (u64)h * dim * rank, rank, n, red);
+  for (int i = wave; i < NB; i += PW) {
     const int bb = b0 + i;
     if (bb >= sv.b) continue;
-    float v = 0.f;
-#pragma unroll
-    for (int g = 0; g < 4; ++g) v += red[(g * NB + i) * 64 + lane];
     T* o = out + ((u64)bb * heads + h) * (rank + rot);
-    if (n < rank) stf(o + n, v);
+    if (n < rank) stf(o + n, head_sum<NB>(red, i, lane));
     if (blockIdx.x == 0) {
       const T* qr = q + ((u64)bb * heads + h) * (dim + rot) + dim;
       const int pos = sv.lens[sv.slots[bb]];
@@ -155,65 +170,56 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(
 }
 
 // part [b, splits, heads, rank + 2] = {sum p c, max, sum p} per key range
-template <typename T>
-__global__ __launch_bounds__(256) void latent_expand_kernel(
+template <typename T, int NB>
+__global__ __launch_bounds__(PTPB) void latent_expand_kernel(
     const float* __restrict__ part, int splits, const float* __restrict__ sink,
     const T* __restrict__ w, const T* __restrict__ g, u64 ldg,
     T* __restrict__ out, int b, int heads, int rank, int vdim) {
   extern __shared__ float sh[];
   float* x = sh;                     // [NB][rank]
-  float* red = sh + NB * rank;       // [4][NB][64]
+  float* red = x + NB * rank;        // [PW][NB][64]
+  float* wt = red + PW * NB * 64;    // [NB][splits]
   const int h = blockIdx.y, b0 = blockIdx.z * NB;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int n = blockIdx.x * 64 + lane;
-  const u64 pr = rank + 2;
-  for (int i = wave; i < NB; i += 4) {
-    const int bb = b0 + i;
-    if (bb >= b) {
-      for (int j = lane; j < rank; j += 64) x[i * rank + j] = 0.f;
-      continue;
-    }
-    const float* p = part + ((u64)bb * splits * heads + h) * pr;
-    const u64 sp = (u64)heads * pr;
+  const u64 pr = rank + 2, sp = (u64)heads * pr;
+  // weight of every key range: the sink joins maximum and denominator
+  for (int i = wave; i < NB; i += PW) {
+    if (b0 + i >= b) continue;
+    const float* p = part + ((u64)(b0 + i) * splits * heads + h) * pr + rank;
     float M = sink[h];
-    for (int c = 0; c < splits; ++c) M = fmaxf(M, p[c * sp + rank]);
-    float L = expf(sink[h] - M);
-    for (int c = 0; c < splits; ++c)
-      L += expf(p[c * sp + rank] - M) * p[c * sp + rank + 1];
-    const float inv = 1.f / L;
-    for (int j = lane; j < rank; j += 64) {
-      float a = 0.f;
-      for (int c = 0; c < splits; ++c)
-        a = fmaf(expf(p[c * sp + rank] - M), p[c * sp + j], a);
-      x[i * rank + j] = a * inv;
+    for (int c = lane; c < splits; c += 64) M = fmaxf(M, p[c * sp]);
+    M = wave_reduce_max(M);
+    float L = 0.f;
+    for (int c = lane; c < splits; c += 64) {
+      const float e = expf(p[c * sp] - M);
+      wt[i * splits + c] = e;
+      L = fmaf(e, p[c * sp + 1], L);
     }
+    L = wave_reduce_sum(L) + expf(sink[h] - M);
+    for (int c = lane; c < splits; c += 64) wt[i * splits + c] /= L;
   }
   __syncthreads();
-  float acc[NB];
-#pragma unroll
-  for (int i = 0; i < NB; ++i) acc[i] = 0.f;
-  if (n < vdim) {
-    const T* wp = w + (u64)h * rank * vdim + n;
+  for (int id = threadIdx.x; id < NB * rank; id += PTPB) {
+    const int i = id / rank, j = id % rank;
+    float a = 0.f;
+    if (b0 + i < b) {
+      const float* p = part + ((u64)(b0 + i) * splits * heads + h) * pr + j;
 #pragma unroll 8
-    for (int k = wave; k < rank; k += 4) {
-      const float wv = ldf(wp + (u64)k * vdim);
-#pragma unroll
-      for (int i = 0; i < NB; ++i) acc[i] = fmaf(x[i * rank + k], wv, acc[i]);
+      for (int c = 0; c < splits; ++c)
+        a = fmaf(wt[i * splits + c], p[c * sp], a);
     }
+    x[id] = a;
   }
-#pragma unroll
-  for (int i = 0; i < NB; ++i) red[(wave * NB + i) * 64 + lane] = acc[i];
   __syncthreads();
+  head_product<T, NB>(x, rank, w + (u64)h * rank * vdim, vdim, n, red);
   if (n >= vdim) return;
-  for (int i = wave; i < NB; i += 4) {
+  for (int i = wave; i < NB; i += PW) {
     const int bb = b0 + i;
     if (bb >= b) continue;
-    float v = 0.f;
-#pragma unroll
-    for (int k = 0; k < 4; ++k) v += red[(k * NB + i) * 64 + lane];
     const u64 c = (u64)h * vdim + n;
     stf(out + (u64)bb * heads * vdim + c,
-        v * sigmoid_f(ldf(g + (u64)bb * ldg + c)));
+        head_sum<NB>(red, i, lane) * sigmoid_f(ldf(g + (u64)bb * ldg + c)));
   }
 }
 
@@ -255,14 +261,20 @@ hipError_t lfmq_latent_absorb(const void* q, const void* w, const SeqView& sv,
                               const void* inv_freq, void* out, int heads,
                               int dim, int rot, int rot_dims, int rank,
                               bool f32, hipStream_t stream) {
-  const dim3 grid((rank + 63) / 64, heads, (sv.b + NB - 1) / NB), block(256);
-  const size_t lds = (NB * (size_t)dim + 4 * NB * 64) * sizeof(float);
+  const int nb = sv.b == 1 ? 1 : (sv.b <= 4 ? 4 : 8);
+  const dim3 grid((rank + 63) / 64, heads, (sv.b + nb - 1) / nb), block(PTPB);
+  const size_t lds = (nb * (size_t)dim + PW * nb * 64) * sizeof(float);
   if (lds > 64 * 1024) return hipErrorInvalidValue;
-#define GO(T)                                                                \
-  hipLaunchKernelGGL(latent_absorb_kernel<T>, grid, block, lds, stream,      \
+#define GO(T, B)                                                             \
+  hipLaunchKernelGGL((latent_absorb_kernel<T, B>), grid, block, lds, stream, \
                      (const T*)q, (const T*)w, sv, (const float*)inv_freq,   \
                      (T*)out, heads, dim, rot, rot_dims, rank)
-  if (f32) GO(float); else GO(bf16_t);
+#define GO2(T)                                                               \
+  do {                                                                       \
+    if (nb == 1) GO(T, 1); else if (nb == 4) GO(T, 4); else GO(T, 8);        \
+  } while (0)
+  if (f32) GO2(float); else GO2(bf16_t);
+#undef GO2
 #undef GO
   return hipGetLastError();
 }
@@ -271,15 +283,22 @@ hipError_t lfmq_latent_expand(const void* part, int splits, const void* sink,
                               const void* w, const void* g, long ldg,
                               void* out, int b, int heads, int rank, int vdim,
                               bool f32, hipStream_t stream) {
-  const dim3 grid((vdim + 63) / 64, heads, (b + NB - 1) / NB), block(256);
-  const size_t lds = (NB * (size_t)rank + 4 * NB * 64) * sizeof(float);
+  const int nb = b == 1 ? 1 : (b <= 4 ? 4 : 8);
+  const dim3 grid((vdim + 63) / 64, heads, (b + nb - 1) / nb), block(PTPB);
+  const size_t lds =
+      (nb * (size_t)rank + PW * nb * 64 + nb * (size_t)splits) * sizeof(float);
   if (lds > 64 * 1024) return hipErrorInvalidValue;
-#define GO(T)                                                                \
-  hipLaunchKernelGGL(latent_expand_kernel<T>, grid, block, lds, stream,      \
+#define GO(T, B)                                                             \
+  hipLaunchKernelGGL((latent_expand_kernel<T, B>), grid, block, lds, stream, \
                      (const float*)part, splits, (const float*)sink,         \
                      (const T*)w, (const T*)g, (u64)ldg, (T*)out, b, heads,  \
                      rank, vdim)
-  if (f32) GO(float); else GO(bf16_t);
+#define GO2(T)                                                               \
+  do {                                                                       \
+    if (nb == 1) GO(T, 1); else if (nb == 4) GO(T, 4); else GO(T, 8);        \
+  } while (0)
+  if (f32) GO2(float); else GO2(bf16_t);
+#undef GO2
 #undef GO
   return hipGetLastError();
 }

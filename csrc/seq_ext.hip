@@ -51,6 +51,10 @@ hipError_t lfmq_attn_window_prompt(const void*, const void*, long, long,
 hipError_t lfmq_attn_window_decode(const void*, const void*, const SeqView&,
                                    void*, int, int, int, int, int, int, float,
                                    bool, hipStream_t);
+bool lfmq_attn_latent_decode_mfma_ok(const void*, const void*, int, int);
+hipError_t lfmq_attn_latent_decode_mfma(const void*, const void*,
+                                        const SeqView&, void*, int, int, int,
+                                        int, int, int, float, hipStream_t);
 bool lfmq_attn_window_prompt_mfma_ok(const void*, const void*, long,
                                      const void*, long, const void*, long, int,
                                      int, int);
@@ -417,7 +421,8 @@ T_ attn_window_prompt(T_ q, T_ kv, T_ lat, T_ seq, T_ cu, T_ slots, T_ lens,
 
 // q [b, H, rank + rot] over the latent ring -> part [b, splits, H, rank + 2]
 T_ attn_window_decode(T_ q, T_ ring, T_ seq, T_ cu, T_ slots, T_ lens,
-                      long rank, long window, long splits, double scale) {
+                      long rank, long window, long splits, double scale,
+                      bool general) {
   const SeqView sv = view(seq, cu, slots, lens);
   const bool f32 = storage(q, "q");
   check(q, q.scalar_type(), "q");
@@ -429,6 +434,15 @@ T_ attn_window_decode(T_ q, T_ ring, T_ seq, T_ cu, T_ slots, T_ lens,
               "attn_window_decode: shape mismatch");
   auto part = torch::empty({sv.b, splits, H, rank + 2},
                            q.options().dtype(torch::kFloat32));
+  if (!f32 && !general &&
+      lfmq_attn_latent_decode_mfma_ok(q.data_ptr(), ring.data_ptr(), (int)rank,
+                                      (int)(D - rank))) {
+    CHECK_HIP(lfmq_attn_latent_decode_mfma(
+        q.data_ptr(), ring.data_ptr(), sv, part.data_ptr(), (int)H, (int)rank,
+        (int)(D - rank), (int)window, (int)ring.size(1), (int)splits,
+        (float)scale, stream()));
+    return part;
+  }
   CHECK_HIP(lfmq_attn_window_decode(q.data_ptr(), ring.data_ptr(), sv,
                                     part.data_ptr(), (int)H, (int)rank,
                                     (int)(D - rank), (int)window,

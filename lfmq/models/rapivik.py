@@ -89,9 +89,9 @@ class RapivikConfig:
                 lat_heads: int, lat_dim: int, rot: int, lat_vdim: int,
                 q_rank: int, kv_rank: int, window: int, vocab: int,
                 n_layers: int, **kw) -> "RapivikConfig":
-        """mLSTM and latent-attention layers in turn, a feed-forward behind
-        the attention."""
-        rec = {"type": "mlstm", "mlp": None,
+        """mLSTM and latent-attention layers in turn, each with a
+        feed-forward."""
+        rec = {"type": "mlstm", "mlp": {"kind": "dense", "ff": ff},
                "mixer": {"heads": heads, "dim": dim, "vdim": vdim,
                          "gate_cap": 15.0}}
         att = {"type": "latent_attention",

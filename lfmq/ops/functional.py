@@ -348,11 +348,13 @@ def attn_window_prompt(q, kv, lat, batch, cache, rows, inv_freq, sink, gate,
 
 
 def attn_window_decode(q, ring, batch, cache, rank: int, window: int,
-                       scale: float) -> torch.Tensor:
-    """Absorbed queries over the latent ring: partial results of a split
-    key range (one token per sequence)."""
+                       scale: float, general: bool = False) -> torch.Tensor:
+    """Absorbed queries over the latent ring (one token per sequence):
+    partial results of a split key range.  general: the any-size kernel
+    also where the matrix-core one applies."""
     reach = min(window, ring.shape[1])
-    # enough key ranges to fill the chip, none shorter than a key tile
-    splits = max(1, min(-(-reach // 64), -(-1024 // (q.shape[0] * q.shape[1]))))
+    # enough key ranges to fill the chip, none shorter than two key tiles
+    groups = -(-q.shape[1] // 32) * q.shape[0]
+    splits = max(1, min(-(-reach // 64), -(-512 // groups), 64))
     return seq_ext().attn_window_decode(q, ring, *batch.view(cache), rank,
-                                        window, splits, scale)
+                                        window, splits, scale, general)

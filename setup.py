@@ -52,6 +52,7 @@ SEQ_SOURCES = [
     "csrc/latent_prep.hip",
     "csrc/attn_window.hip",
     "csrc/attn_window_mfma.hip",
+    "csrc/attn_latent_mfma.hip",
     "csrc/elementwise.hip",
     "csrc/sample.hip",
 ]
