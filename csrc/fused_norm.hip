@@ -99,7 +99,7 @@ __global__ __launch_bounds__(512) void add_norm_kernel(
   }
 }
 
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     const float* __restrict__ o, const T* __restrict__ g, u64 ldg,
     const float* __restrict__ w, T* __restrict__ out, u64 pairs, int heads,
@@ -110,14 +110,27 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
   const u64 row = id / heads;
   const int h = id % heads;
   const float* src = o + id * v;
+  const T* gr = g + row * ldg + h * v;
+  T* dst = out + id * v;
   float ss = 0.f;
-  for (int j = lane; j < v; j += LFMQ_WAVE) ss = fmaf(src[j], src[j], ss);
+#pragma unroll 2
+  for (int j = lane * VEC; j < v; j += LFMQ_WAVE * VEC) {
+    float a[VEC];
+    ldv<float, VEC>(src + j, a);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss = fmaf(a[e], a[e], ss);
+  }
   ss = wave_reduce_sum(ss);
   const float inv = 1.f / sqrtf(ss / (float)v + eps);
-  for (int j = lane; j < v; j += LFMQ_WAVE) {
-    const int c = h * v + j;
-    stf(out + row * heads * v + c,
-        src[j] * inv * w[c] * sigmoid_f(ldf(g + row * ldg + c)));
+#pragma unroll 2
+  for (int j = lane * VEC; j < v; j += LFMQ_WAVE * VEC) {
+    float a[VEC], c[VEC], k[VEC];
+    ldv<float, VEC>(src + j, a);
+    ldv<T, VEC>(gr + j, c);
+    ldv<float, VEC>(w + h * v + j, k);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) a[e] = a[e] * inv * k[e] * sigmoid_f(c[e]);
+    stv<T, VEC>(dst + j, a);
   }
 }
 
@@ -159,11 +172,14 @@ hipError_t lfmq_head_norm_gate(const void* o, const void* g, long ldg,
                                hipStream_t stream) {
   const u64 pairs = (u64)rows * heads;
   const dim3 grid((u32)((pairs + 3) / 4)), block(256);
-#define GO(T)                                                                \
-  hipLaunchKernelGGL(head_norm_gate_kernel<T>, grid, block, 0, stream,       \
+  const bool v4 = v % 4 == 0 && ldg % 4 == 0 &&
+                  (((u64)o | (u64)g | (u64)w | (u64)out) & 15) == 0;
+#define GO(T, V)                                                             \
+  hipLaunchKernelGGL((head_norm_gate_kernel<T, V>), grid, block, 0, stream,  \
                      (const float*)o, (const T*)g, (u64)ldg,                 \
                      (const float*)w, (T*)out, pairs, heads, v, eps)
-  if (f32) GO(float); else GO(bf16_t);
+  if (f32) { if (v4) GO(float, 4); else GO(float, 1); }
+  else { if (v4) GO(bf16_t, 4); else GO(bf16_t, 1); }
 #undef GO
   return hipGetLastError();
 }

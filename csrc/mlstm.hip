@@ -24,38 +24,46 @@ namespace {
 
 constexpr int TPB = 256;
 
-template <typename T, int EPT>
+// C columns and EPT rows of the slice a thread; lanes run over the columns
+// first, so that the sum over rows is a few shuffles and one LDS pass
+template <typename T, int EPT, int C>
 __global__ __launch_bounds__(TPB) void mlstm_scan_kernel(
     const T* __restrict__ qkv, u64 ld, const float* __restrict__ gates,
     SeqView sv, const i32* __restrict__ turn, float* __restrict__ S,
     float* __restrict__ nm, float* __restrict__ out, int heads, int dim,
-    int vdim, float cap, int vs_log2) {
+    int vdim, float cap, int lanes_log2) {
   extern __shared__ float sh[];
-  const int VS = 1 << vs_log2;
-  const int DG = TPB >> vs_log2;
+  const int VL = 1 << lanes_log2;            // threads across the slice
+  const int VS = VL * C, DG = TPB >> lanes_log2;
   float* qs = sh;                 // [2][dim]
   float* ks = sh + 2 * dim;       // [2][dim]
-  float* red = sh + 4 * dim;      // [TPB]
-  float* redn = red + TPB;        // [DG]
+  float* red = sh + 4 * dim;      // [4 waves][VS]
+  float* redn = red + 4 * VS;     // [4]
   const int s = blockIdx.z, h = blockIdx.y;
   const int n0 = sv.cu[s], n1 = sv.cu[s + 1];
   if (n1 <= n0) return;
   const int slot = sv.slots[s];
   const bool fresh = sv.lens[slot] == 0;
   const int cur = turn[slot] & 1;
-  const int vl = threadIdx.x & (VS - 1), dg = threadIdx.x >> vs_log2;
-  const int v = blockIdx.x * VS + vl;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int vl = threadIdx.x & (VL - 1), dg = threadIdx.x >> lanes_log2;
+  const int v = blockIdx.x * VS + vl * C;    // C divides vdim
   const bool vok = v < vdim;
   const u64 sh_base = ((u64)slot * heads + h) * dim;
   float* Sp = S + sh_base * vdim;
   const float* nm_in = nm + (((u64)slot * 2 + cur) * heads + h) * (dim + 1);
   float* nm_out = nm + (((u64)slot * 2 + (cur ^ 1)) * heads + h) * (dim + 1);
 
-  float st[EPT], nn[EPT];
+  float st[EPT][C], nn[EPT];
 #pragma unroll
   for (int e = 0; e < EPT; ++e) {
     const int d = dg + DG * e;
-    st[e] = (!fresh && d < dim && vok) ? Sp[(u64)d * vdim + v] : 0.f;
+    if (!fresh && d < dim && vok) {
+      ldv<float, C>(Sp + (u64)d * vdim + v, st[e]);
+    } else {
+#pragma unroll
+      for (int c = 0; c < C; ++c) st[e][c] = 0.f;
+    }
     nn[e] = (!fresh && d < dim) ? nm_in[d] : 0.f;
   }
   float m = fresh ? 0.f : nm_in[dim];
@@ -72,7 +80,9 @@ __global__ __launch_bounds__(TPB) void mlstm_scan_kernel(
       q[d] = ldf(r + d) * qscale;
       k[d] = ldf(r + koff + d);
     }
-    const float vv = vok ? ldf(r + voff + v) : 0.f;
+    float vv[C];
+#pragma unroll
+    for (int c = 0; c < C; ++c) vv[c] = vok ? ldf(r + voff + v + c) : 0.f;
     const float gi = mlstm_input_gate(gates[(u64)row * 2 * heads + h], cap);
     const float gf =
         mlstm_forget_gate(gates[(u64)row * 2 * heads + heads + h], cap);
@@ -80,34 +90,46 @@ __global__ __launch_bounds__(TPB) void mlstm_scan_kernel(
     const float a = expf(gf + m - m2), b = expf(gi - m2);
     m = m2;
     __syncthreads();   // q, k staged; the last token's red is consumed
-    float acc = 0.f, den = 0.f;
+    float acc[C] = {}, den = 0.f;
 #pragma unroll
     for (int e = 0; e < EPT; ++e) {
       const int d = dg + DG * e;
       const bool ok = d < dim;
       const float kd = ok ? k[d] : 0.f, qd = ok ? q[d] : 0.f;
-      st[e] = fmaf(a, st[e], b * kd * vv);
-      nn[e] = fmaf(a, nn[e], b * kd);
-      acc = fmaf(st[e], qd, acc);
+      const float bk = b * kd;
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        st[e][c] = fmaf(a, st[e][c], bk * vv[c]);
+        acc[c] = fmaf(st[e][c], qd, acc[c]);
+      }
+      nn[e] = fmaf(a, nn[e], bk);
       den = fmaf(nn[e], qd, den);
     }
-    red[threadIdx.x] = acc;
-    if (vl == 0) redn[dg] = den;
+    for (int o = VL; o < 64; o <<= 1) {
+#pragma unroll
+      for (int c = 0; c < C; ++c) acc[c] += __shfl_xor(acc[c], o, 64);
+      den += __shfl_xor(den, o, 64);
+    }
+    if (lane < VL) {
+#pragma unroll
+      for (int c = 0; c < C; ++c) red[wave * VS + lane * C + c] = acc[c];
+    }
+    if (lane == 0) redn[wave] = den;
     __syncthreads();
-    if (dg == 0 && vok) {
-      float num = 0.f, dn = 0.f;
-      for (int g = 0; g < DG; ++g) {
-        num += red[g * VS + vl];
-        dn += redn[g];
-      }
-      out[((u64)row * heads + h) * vdim + v] =
+    const int vo = blockIdx.x * VS + threadIdx.x;
+    if (threadIdx.x < VS && vo < vdim) {
+      float num = 0.f;
+#pragma unroll
+      for (int w = 0; w < TPB / 64; ++w) num += red[w * VS + threadIdx.x];
+      const float dn = redn[0] + redn[1] + redn[2] + redn[3];
+      out[((u64)row * heads + h) * vdim + vo] =
           num / (fmaxf(fabsf(dn), expf(-m)) + 1e-6f);
     }
   }
 #pragma unroll
   for (int e = 0; e < EPT; ++e) {
     const int d = dg + DG * e;
-    if (d < dim && vok) Sp[(u64)d * vdim + v] = st[e];
+    if (d < dim && vok) stv<float, C>(Sp + (u64)d * vdim + v, st[e]);
     if (d < dim && vl == 0 && blockIdx.x == 0) nm_out[d] = nn[e];
   }
   if (threadIdx.x == 0 && blockIdx.x == 0) nm_out[dim] = m;
@@ -119,28 +141,39 @@ hipError_t lfmq_mlstm_scan(const void* qkv, long ld, const void* gates,
                            const SeqView& sv, const void* turn, void* S,
                            void* nm, void* out, int heads, int dim, int vdim,
                            float cap, bool f32, hipStream_t stream) {
-  // narrow value slices give more workgroups; wide ones longer rows
-  int vl = 6;
-  while (vl > 4 && ((u64)sv.b * heads * ((vdim + (1 << vl) - 1) >> vl) < 1024 ||
-                    dim > (TPB >> vl) * 64))
-    --vl;
-  const int dg = TPB >> vl;
+  const int c = vdim % 4 == 0 ? 4 : 1;
+  const int max_ept = c == 4 ? 16 : 64;
+  // narrow slices give more workgroups, wide ones longer rows
+  int vs = 64;
+  while (vs > 16 &&
+         ((u64)sv.b * heads * ((vdim + vs - 1) / vs) < 1024 ||
+          dim > TPB * c / vs * max_ept))
+    vs /= 2;
+  int lanes_log2 = 0;
+  while ((c << lanes_log2) < vs) ++lanes_log2;
+  const int dg = TPB >> lanes_log2;
   const int ept = (dim + dg - 1) / dg;
-  if (ept > 64) return hipErrorInvalidValue;
-  const dim3 grid((vdim + (1 << vl) - 1) >> vl, heads, sv.b), block(TPB);
-  const size_t lds = (4 * (size_t)dim + TPB + dg) * sizeof(float);
-#define GO(T, E)                                                             \
-  hipLaunchKernelGGL((mlstm_scan_kernel<T, E>), grid, block, lds, stream,    \
+  if (ept > max_ept) return hipErrorInvalidValue;
+  const dim3 grid((vdim + vs - 1) / vs, heads, sv.b), block(TPB);
+  const size_t lds = (4 * (size_t)dim + 4 * vs + 4) * sizeof(float);
+#define GO(T, E, C)                                                          \
+  hipLaunchKernelGGL((mlstm_scan_kernel<T, E, C>), grid, block, lds, stream, \
                      (const T*)qkv, (u64)ld, (const float*)gates, sv,        \
                      (const i32*)turn, (float*)S, (float*)nm, (float*)out,   \
-                     heads, dim, vdim, cap, vl)
+                     heads, dim, vdim, cap, lanes_log2)
 #define GO2(T)                                                               \
   do {                                                                       \
-    if (ept <= 4) GO(T, 4);                                                  \
-    else if (ept <= 8) GO(T, 8);                                             \
-    else if (ept <= 16) GO(T, 16);                                           \
-    else if (ept <= 32) GO(T, 32);                                           \
-    else GO(T, 64);                                                          \
+    if (c == 4) {                                                            \
+      if (ept <= 1) GO(T, 1, 4);                                             \
+      else if (ept <= 2) GO(T, 2, 4);                                        \
+      else if (ept <= 4) GO(T, 4, 4);                                        \
+      else if (ept <= 8) GO(T, 8, 4);                                        \
+      else GO(T, 16, 4);                                                     \
+    } else {                                                                 \
+      if (ept <= 8) GO(T, 8, 1);                                             \
+      else if (ept <= 16) GO(T, 16, 1);                                      \
+      else GO(T, 64, 1);                                                     \
+    }                                                                        \
   } while (0)
   if (f32) GO2(float); else GO2(bf16_t);
 #undef GO2

@@ -12,8 +12,8 @@
 //   S_c+1 = exp(F_L + m_c - m_L) S_c + sum_s exp(F_L - F_s + i_s - m_L) k_s v_s^T
 //
 // Three kernels:
-//   gates   scan of (F, m) per head: (+, max) composition over 256 tokens
-//           at a time
+//   gates   scan of (F, m) per head: (+, max) composition over 1024
+//           tokens at a time
 //   states  S and n at every chunk start.  A workgroup owns a 64 x 64 tile
 //           of S in accumulators and walks the sequence, the next tokens'
 //           rows in flight while it multiplies
@@ -33,7 +33,9 @@ namespace {
 __device__ __forceinline__ u32 swz(u32 row) { return (row ^ (row >> 3)) & 7; }
 
 // ---- gates ---------------------------------------------------------------
-__global__ __launch_bounds__(256) void mlstm_gate_scan_kernel(
+constexpr int GT = 1024, GW = GT / 64;
+
+__global__ __launch_bounds__(GT) void mlstm_gate_scan_kernel(
     const float* __restrict__ gates, SeqView sv, const i32* __restrict__ turn,
     float* __restrict__ nm, float* __restrict__ gF, float* __restrict__ gI,
     float* __restrict__ gM, int heads, int dim, float cap, int waves_per_chunk) {
@@ -45,13 +47,22 @@ __global__ __launch_bounds__(256) void mlstm_gate_scan_kernel(
   const u64 st = (u64)heads * (dim + 1), at = (u64)h * (dim + 1) + dim;
   float m = fresh ? 0.f : nm[((u64)slot * 2 + cur) * st + at];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  __shared__ float wF[4], wM[4];
-  for (int b0 = n0; b0 < n1; b0 += 256) {
+  __shared__ float wF[GW], wM[GW];
+  float ri = 0.f, rf = 0.f;                  // raw gates, one block ahead
+  auto fetch = [&](int row) {
+    if (row < n1) {
+      const float* g = gates + (u64)row * 2 * heads + h;
+      ri = g[0];
+      rf = g[heads];
+    }
+  };
+  fetch(n0 + threadIdx.x);
+  for (int b0 = n0; b0 < n1; b0 += GT) {
     const int row = b0 + threadIdx.x;
     const bool live = row < n1;
-    const float* g = gates + (u64)row * 2 * heads + h;
-    const float gi = live ? mlstm_input_gate(g[0], cap) : -INFINITY;
-    float F = live ? mlstm_forget_gate(g[heads], cap) : 0.f;
+    const float gi = live ? mlstm_input_gate(ri, cap) : -INFINITY;
+    float F = live ? mlstm_forget_gate(rf, cap) : 0.f;
+    fetch(row + GT);
     float M = gi;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -67,7 +78,7 @@ __global__ __launch_bounds__(256) void mlstm_gate_scan_kernel(
     }
     __syncthreads();
     float mc = m, Floc = F;
-    for (int w = 0; w < 4; ++w) {
+    for (int w = 0; w < GW; ++w) {
       if (w < wave) {
         mc = fmaxf(wF[w] + mc, wM[w]);
         if (w >= wave - wave % waves_per_chunk) Floc += wF[w];
@@ -583,7 +594,7 @@ hipError_t lfmq_mlstm_chunk(const void* qkv, long ld, const void* gates,
           (unsigned short*)ws, (float*)nws, (const float*)norm_w,
           (bf16_t*)out, heads, dim, vdim, L, (dim + 63) / 64 * 64,
           (vdim + 63) / 64 * 64, eps};
-  hipLaunchKernelGGL(mlstm_gate_scan_kernel, dim3(heads, sv.b), dim3(256), 0,
+  hipLaunchKernelGGL(mlstm_gate_scan_kernel, dim3(heads, sv.b), dim3(GT), 0,
                      stream, (const float*)gates, sv, (const i32*)turn,
                      (float*)nm, g, g + hn, g + 2 * hn, heads, dim, cap,
                      L / 64);

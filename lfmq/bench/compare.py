@@ -78,8 +78,9 @@ def compare(size: str, n_layers: int, steps: int = 64, repeats: int = 3,
             prefill=PREFILL, decode=DECODE):
     """Yields one dict per (phase, shape) with both models' tokens/s."""
     models = {k: _build(f(n_layers), "cuda") for k, f in SIZES[size].items()}
-    params = {k: sum(p.numel() for p in m.parameters()) / 1e6
-              for k, m in models.items()}
+    params = {k: sum(p.numel() for n, p in m.named_parameters()
+                     if not n.startswith(("embed", "bigram", "lm_head"))) / 1e6
+              for k, m in models.items()}          # of the layers
     for phase, shapes in (("prefill", prefill), ("decode", decode)):
         for b, s in shapes:
             row = {"size": size, "layers": n_layers, "phase": phase,

@@ -36,6 +36,11 @@ def _bench_config(model_name: str, n_layers: Optional[int] = None):
     elif model_name == "mixtral-8x7b":
         from ..models.mixtral import MixtralConfig
         cfg = MixtralConfig.mixtral_8x7b()
+    elif model_name in ("rapivik-1b", "rapivik-8b", "tiny-rapivik"):
+        from ..models.rapivik import RapivikConfig
+        cfg = {"rapivik-1b": RapivikConfig.sized_1b,
+               "rapivik-8b": RapivikConfig.sized_8b,
+               "tiny-rapivik": RapivikConfig.tiny}[model_name]()
     elif model_name == "tiny-debug":
         # contract-test shape only (tests/test_bench_contract.py);
         # never a reportable benchmark config
