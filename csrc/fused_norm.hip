@@ -4,8 +4,8 @@
 // h = x * rsqrt(mean(x^2) + eps) * (bias + w) in one pass over the row,
 // with an optional SIDE PROJECTION p = h * Wp^T + bp of a few outputs in
 // fp32 (the gates of a recurrent layer must not round to 16 bits, and the
-// row is in LDS already).  bias 1 gives the weight-around-zero norm, bias
-// 0 the plain one.
+// row is in LDS already).  bias 1 is for weights kept as offsets from one,
+// bias 0 for plain ones.
 //
 // One wave owns a row; a workgroup takes `rpw` rows, so that the side
 // projection's weights are read once for all of them.  With one row per
