@@ -5,11 +5,12 @@
 // Query row r of sequence s at position p sees keys j with
 // p - window < j <= p.  A key is {k1 [d1] per head, k2 [d2] shared by all
 // heads}, its value [dv] per head; strides of 0 share a part between
-// heads.  Key rows come from a packed step buffer (row = own_row[s] + j -
-// len0) or, with own_row null, from a ring cache (slot * cap + j mod cap).
+// heads, and `group` query heads share a key/value head.  Key rows come
+// from a packed step buffer (row = own_row[s] + j - len0) or, with own_row
+// null, from a ring cache (slot * cap + j mod cap).
 //
-// PROMPT: rotates the query's second part, applies the sink and the output
-// gate, writes 16/32-bit rows.  DECODE (absorbed latent form): takes a
+// PROMPT: rotates the query's second part, applies the sink, an output
+// gate if there is one and a constant gain, writes 16/32-bit rows.  DECODE (absorbed latent form): takes a
 // ready query, emits the partial {sum p v, max, sum p} of one key range.
 #include "seq_common.h"
 
@@ -22,6 +23,9 @@ struct WinArgs {
   int heads, d1, d2, rot_dims, dv, window, cap, splits;
   float scale;
   u64 k1_ld, k1_head, k2_ld, v_ld, v_head, ldg;
+  int group;
+  u64 ldo;
+  float gain;
 };
 
 template <typename T, bool DECODE>
@@ -37,7 +41,7 @@ __global__ __launch_bounds__(TPB) void attn_window_kernel(
   float* acc = qs + D;            // [dv]
   float* ps = acc + A.dv;         // [KT]
   __shared__ float red[4];
-  const int row = blockIdx.x, h = blockIdx.y;
+  const int row = blockIdx.x, h = blockIdx.y, kh = h / A.group;
   const int s = sv.seq[row];
   const int slot = sv.slots[s];
   const int len0 = sv.lens[slot];
@@ -58,7 +62,7 @@ __global__ __launch_bounds__(TPB) void attn_window_kernel(
     }
     __syncthreads();
   }
-  int lo = max(0, pos - A.window + 1), hi = pos + 1;
+  int lo = pos < A.window ? 0 : pos - A.window + 1, hi = pos + 1;
   if (DECODE) {   // this workgroup's share of the window
     const int per = (hi - lo + A.splits - 1) / A.splits;
     lo += blockIdx.z * per;
@@ -72,7 +76,7 @@ __global__ __launch_bounds__(TPB) void attn_window_kernel(
       const int j = t0 + i;
       const u64 kr = own_row != nullptr ? (u64)(own_row[s] + j - len0)
                                         : (u64)slot * A.cap + j % A.cap;
-      const T* a = k1 + kr * A.k1_ld + h * A.k1_head;
+      const T* a = k1 + kr * A.k1_ld + kh * A.k1_head;
       const T* b = k2 + kr * A.k2_ld;
       float d = 0.f;
       for (int e = lane; e < A.d1; e += 64) d = fmaf(ldf(a + e), qs[e], d);
@@ -103,7 +107,7 @@ __global__ __launch_bounds__(TPB) void attn_window_kernel(
         const int j = t0 + i;
         const u64 kr = own_row != nullptr ? (u64)(own_row[s] + j - len0)
                                           : (u64)slot * A.cap + j % A.cap;
-        o = fmaf(ps[i], ldf(vv + kr * A.v_ld + h * A.v_head + e), o);
+        o = fmaf(ps[i], ldf(vv + kr * A.v_ld + kh * A.v_head + e), o);
       }
       acc[e] = o;
     }
@@ -120,11 +124,12 @@ __global__ __launch_bounds__(TPB) void attn_window_kernel(
     return;
   }
   const float M = fmaxf(m, sink[h]);
-  const float w = expf(m - M) / (l * expf(m - M) + expf(sink[h] - M));
-  T* o = (T*)outp + ((u64)row * A.heads + h) * A.dv;
+  const float w =
+      A.gain * expf(m - M) / (l * expf(m - M) + expf(sink[h] - M));
+  T* o = (T*)outp + (u64)row * A.ldo + h * A.dv;
   const T* gr = g + (u64)row * A.ldg + h * A.dv;
   for (int e = threadIdx.x; e < A.dv; e += TPB)
-    stf(o + e, acc[e] * w * sigmoid_f(ldf(gr + e)));
+    stf(o + e, acc[e] * w * (g != nullptr ? sigmoid_f(ldf(gr + e)) : 1.f));
 }
 
 }  // namespace
@@ -138,7 +143,8 @@ hipError_t lfmq_attn_window_prompt(
     int rot_dims, int dv, int window, float scale, bool f32,
     hipStream_t stream) {
   WinArgs A{heads, d1, d2, rot_dims, dv, window, 0, 1, scale, (u64)k1_ld,
-            (u64)k1_head, (u64)k2_ld, (u64)v_ld, (u64)v_head, (u64)ldg};
+            (u64)k1_head, (u64)k2_ld, (u64)v_ld, (u64)v_head, (u64)ldg, 1,
+            (u64)heads * dv, 1.f};
   const size_t lds = (size_t)(d1 + d2 + dv + KT) * sizeof(float);
   if (lds > 60 * 1024) return hipErrorInvalidValue;
 #define GO(T)                                                                \
@@ -161,7 +167,7 @@ hipError_t lfmq_attn_window_decode(const void* q, const void* ring,
                                    hipStream_t stream) {
   const u64 d = rank + rot;
   WinArgs A{heads, rank, rot, 0, rank, window, cap, splits, scale,
-            d, 0, d, d, 0, 0};
+            d, 0, d, d, 0, 0, 1, 0, 1.f};
   const size_t lds = (size_t)(d + rank + KT) * sizeof(float);
   if (lds > 60 * 1024) return hipErrorInvalidValue;
 #define GO(T)                                                                \
@@ -171,6 +177,30 @@ hipError_t lfmq_attn_window_decode(const void* q, const void* ring,
                      (const T*)ring, sv, (const i32*)nullptr,                \
                      (const float*)nullptr, (const float*)nullptr,           \
                      (const T*)nullptr, part, A)
+  if (f32) GO(float); else GO(bf16_t);
+#undef GO
+  return hipGetLastError();
+}
+
+// grouped queries over a key/value cache: kc [slots, cap, heads / group,
+// dim], vc [.., dv]; q [n, heads, dim] ready; out rows of stride ldo.
+// Every position from 0 on is seen; any number of tokens per sequence.
+hipError_t lfmq_attn_grouped(const void* q, const void* kc, const void* vc,
+                             const SeqView& sv, const void* sink, void* out,
+                             long ldo, int heads, int group, int dim, int dv,
+                             int cap, float scale, float gain, bool f32,
+                             hipStream_t stream) {
+  const u64 kv = heads / group;
+  WinArgs A{heads, dim, 0, 0, dv, INT32_MAX, cap, 1, scale, kv * dim,
+            (u64)dim, 0, kv * dv, (u64)dv, 0, group, (u64)ldo, gain};
+  const size_t lds = (size_t)(dim + dv + KT) * sizeof(float);
+  if (lds > 60 * 1024) return hipErrorInvalidValue;
+#define GO(T)                                                                \
+  hipLaunchKernelGGL((attn_window_kernel<T, false>), dim3(sv.n, heads),      \
+                     dim3(TPB), lds, stream, (const T*)q, (const T*)kc,      \
+                     (const T*)kc, (const T*)vc, sv, (const i32*)nullptr,    \
+                     (const float*)nullptr, (const float*)sink,              \
+                     (const T*)nullptr, out, A)
   if (f32) GO(float); else GO(bf16_t);
 #undef GO
   return hipGetLastError();

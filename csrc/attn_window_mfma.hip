@@ -24,6 +24,9 @@ struct PArgs {
   bf16_t* out;
   int heads, d1, d2, rot_dims, dv, window;
   float scale;
+  int group, cap;        // query heads a key/value head; cache rows a slot
+  u64 ldo;
+  float gain;
 };
 
 __device__ __forceinline__ u32 swz(u32 row) { return (row ^ (row >> 3)) & 7; }
@@ -37,10 +40,12 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
   char* ldsK = smem;
   char* ldsV = ldsK + BN * KROW;
   char* ldsP = ldsV + VP * 128;
-  const int s = blockIdx.z, h = blockIdx.y, q0 = blockIdx.x * BM;
+  // the last queries see the most keys: they start first
+  const int q0 = (gridDim.x - 1 - blockIdx.x) * BM;
+  const int s = blockIdx.z, h = blockIdx.y, kh = h / A.group;
   const int row0 = sv.cu[s], cnt = sv.cu[s + 1] - row0;
   if (q0 >= cnt) return;
-  const int len0 = sv.lens[sv.slots[s]];
+  const int slot = sv.slots[s], len0 = sv.lens[slot];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int l15 = lane & 15, l4 = lane >> 4;
   const int D = A.d1 + A.d2;
@@ -77,8 +82,10 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
   f32x4 oacc[VT] = {};
 
   const int p_lo = len0 + q0, p_hi = len0 + min(q0 + BM, cnt) - 1;
-  const int lo = max(0, p_lo - A.window + 1), hi = p_hi + 1;
-  const long base = (long)A.own_row[s] - len0;   // buffer row of key 0
+  const int lo = p_lo < A.window ? 0 : p_lo - A.window + 1, hi = p_hi + 1;
+  // row of key 0: in the step's key buffer, or in the cache
+  const long base = A.own_row != nullptr ? (long)A.own_row[s] - len0
+                                         : (long)slot * A.cap;
   for (int t0 = lo; t0 < hi; t0 += BN) {
     __syncthreads();
 #pragma unroll 4
@@ -87,7 +94,7 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
       const u64 kr = (u64)(base + min(t0 + key, hi - 1));
       u32x4 d = {0, 0, 0, 0};
       if (e0 < A.d1)
-        d = *(const u32x4*)(A.k1 + kr * A.k1_ld + h * A.d1 + e0);
+        d = *(const u32x4*)(A.k1 + kr * A.k1_ld + kh * A.d1 + e0);
       else if (e0 < D)
         d = *(const u32x4*)(A.k2 + kr * A.k2_ld + (e0 - A.d1));
       *(u32x4*)(ldsK + key * KROW + e0 * 2) = d;
@@ -99,8 +106,8 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
       if (dg * 8 < A.dv) {
         const u64 ra = (u64)(base + min(t0 + 2 * kp, hi - 1));
         const u64 rb = (u64)(base + min(t0 + 2 * kp + 1, hi - 1));
-        a = *(const u32x4*)(A.v + ra * A.v_ld + h * A.dv + dg * 8);
-        b = *(const u32x4*)(A.v + rb * A.v_ld + h * A.dv + dg * 8);
+        a = *(const u32x4*)(A.v + ra * A.v_ld + kh * A.dv + dg * 8);
+        b = *(const u32x4*)(A.v + rb * A.v_ld + kh * A.dv + dg * 8);
       }
       const u32 blk = kp >> 2, off = (kp & 3) * 4;
 #pragma unroll
@@ -129,7 +136,7 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int pos = p_lo + wave * 16 + l4 * 4 + r;
-        const bool ok = j <= pos && j > pos - A.window && j < hi;
+        const bool ok = j <= pos && pos - j < A.window && j < hi;
         sc[nt][r] = ok ? sc[nt][r] * A.scale : -INFINITY;
       }
     }
@@ -182,14 +189,16 @@ __global__ __launch_bounds__(TPB) void attn_window_prompt_mfma(SeqView sv,
   for (int r = 0; r < 4; ++r) {
     const int qr = q0 + wave * 16 + l4 * 4 + r;
     if (qr >= cnt) continue;
-    const float inv = 1.f / lrun[r];
+    const float inv = A.gain / lrun[r];
     const u64 row = row0 + qr;
     const bf16_t* gr = A.g + row * A.ldg + h * A.dv;
-    bf16_t* o = A.out + (row * A.heads + h) * A.dv;
+    bf16_t* o = A.out + row * A.ldo + h * A.dv;
 #pragma unroll
     for (int on = 0; on < VT; ++on) {
       const int e = on * 16 + l15;
-      if (e < A.dv) stf(o + e, oacc[on][r] * inv * sigmoid_f(ldf(gr + e)));
+      if (e < A.dv)
+        stf(o + e, oacc[on][r] * inv *
+                       (A.g != nullptr ? sigmoid_f(ldf(gr + e)) : 1.f));
     }
   }
 }
@@ -210,6 +219,24 @@ hipError_t launch(const SeqView& sv, const PArgs& A, int max_count,
                      dim3((max_count + BM - 1) / BM, A.heads, sv.b),
                      dim3(TPB), lds, stream, sv, A);
   return hipGetLastError();
+}
+
+hipError_t dispatch(const SeqView& sv, const PArgs& A, int max_count,
+                    hipStream_t stream) {
+  const int ks = (A.d1 + A.d2 + 31) / 32, vt = (A.dv + 15) / 16;
+#define GO(K, V) return launch<K, V>(sv, A, max_count, stream)
+#define GOV(K)                                                               \
+  do {                                                                       \
+    if (vt <= 4) GO(K, 4);                                                   \
+    if (vt <= 8) GO(K, 8);                                                   \
+    GO(K, 16);                                                               \
+  } while (0)
+  if (ks <= 2) GOV(2);
+  if (ks <= 4) GOV(4);
+  if (ks <= 6) GOV(6);
+  GOV(8);
+#undef GOV
+#undef GO
 }
 
 bool al16(const void* p) { return ((u64)p & 15) == 0; }
@@ -236,19 +263,28 @@ hipError_t lfmq_attn_window_prompt_mfma(
           (const bf16_t*)v, (const bf16_t*)g, (u64)k1_ld, (u64)k2_ld,
           (u64)v_ld, (u64)ldg, (const i32*)own_row, (const float*)inv_freq,
           (const float*)sink, (bf16_t*)out, heads, d1, d2, rot_dims, dv,
-          window, scale};
-  const int ks = (d1 + d2 + 31) / 32, vt = (dv + 15) / 16;
-#define GO(K, V) return launch<K, V>(sv, A, max_count, stream)
-#define GOV(K)                                                               \
-  do {                                                                       \
-    if (vt <= 4) GO(K, 4);                                                   \
-    if (vt <= 8) GO(K, 8);                                                   \
-    GO(K, 16);                                                               \
-  } while (0)
-  if (ks <= 2) GOV(2);
-  if (ks <= 4) GOV(4);
-  if (ks <= 6) GOV(6);
-  GOV(8);
-#undef GOV
-#undef GO
+          window, scale, 1, 0, (u64)heads * dv, 1.f};
+  return dispatch(sv, A, max_count, stream);
+}
+
+// grouped queries over a key/value cache (attn_window.hip:
+// lfmq_attn_grouped)
+bool lfmq_attn_grouped_mfma_ok(const void* q, const void* kc, const void* vc,
+                               int dim, int dv) {
+  return dim % 8 == 0 && dv % 8 == 0 && dim <= 256 && dv <= 256 && al16(q) &&
+         al16(kc) && al16(vc);
+}
+
+hipError_t lfmq_attn_grouped_mfma(const void* q, const void* kc,
+                                  const void* vc, const SeqView& sv,
+                                  const void* sink, void* out, long ldo,
+                                  int heads, int group, int dim, int dv,
+                                  int cap, float scale, float gain,
+                                  int max_count, hipStream_t stream) {
+  const u64 kv = heads / group;
+  PArgs A{(const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)kc,
+          (const bf16_t*)vc, nullptr, kv * dim, 0, kv * dv, 0, nullptr,
+          nullptr, (const float*)sink, (bf16_t*)out, heads, dim, 0, 0, dv,
+          INT32_MAX, scale, group, cap, (u64)ldo, gain};
+  return dispatch(sv, A, max_count, stream);
 }

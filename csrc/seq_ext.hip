@@ -1,6 +1,6 @@
 // lfmq_seq — torch bindings of the sequence-mixing layers' kernels (packed
-// variable-length batches, recurrent states, windowed latent attention)
-// and of the small ops every model shares.  Every entry checks dtypes,
+// variable-length batches, recurrent states, latent and grouped attention,
+// experts) and of the small ops every model shares.  Every entry checks dtypes,
 // devices and the sizes that its kernel and grid assume; no fallbacks.
 #include <torch/extension.h>
 #include <ATen/cuda/CUDAContext.h>
@@ -62,6 +62,49 @@ hipError_t lfmq_attn_window_prompt_mfma(
     const void*, const void*, long, const void*, long, const void*, long,
     const SeqView&, const void*, const void*, const void*, const void*, long,
     void*, int, int, int, int, int, int, float, int, hipStream_t);
+hipError_t lfmq_post_norm(void*, const void*, const void*, const void*, void*,
+                          int, int, float, float, bool, hipStream_t);
+hipError_t lfmq_embed_norm(void*, const void*, const void*, const void*,
+                           void*, int, int, int, float, bool, hipStream_t);
+hipError_t lfmq_post_norm_experts(void*, const void*, const void*, int,
+                                  const void*, const void*, const void*,
+                                  const void*, void*, int, int, float, float,
+                                  bool, hipStream_t);
+hipError_t lfmq_qk_prep(const void*, long, const SeqView&, const void*,
+                        const void*, const void*, void*, void*, void*, int,
+                        int, int, int, int, int, float, bool, hipStream_t);
+hipError_t lfmq_attn_grouped(const void*, const void*, const void*,
+                             const SeqView&, const void*, void*, long, int,
+                             int, int, int, int, float, float, bool,
+                             hipStream_t);
+bool lfmq_attn_grouped_mfma_ok(const void*, const void*, const void*, int,
+                               int);
+hipError_t lfmq_attn_grouped_mfma(const void*, const void*, const void*,
+                                  const SeqView&, const void*, void*, long,
+                                  int, int, int, int, int, float, float, int,
+                                  hipStream_t);
+int lfmq_attn_grouped_splits(int, int, int, int);
+hipError_t lfmq_attn_grouped_decode(const void*, const void*, const void*,
+                                    const SeqView&, const void*, void*, void*,
+                                    long, int, int, int, int, int, int, float,
+                                    float, hipStream_t);
+bool lfmq_lru_mfma_ok(const void*, int);
+hipError_t lfmq_gated_lru(const SeqView&, const void*, const void*, long,
+                          const void*, const void*, const void*, const void*,
+                          const void*, const void*, const void*, void*, void*,
+                          void*, long, int, int, int, float, float, void*,
+                          void*, void*, const void*, int, bool, bool, bool,
+                          hipStream_t);
+hipError_t lfmq_moe_route_sort(const void*, const void*, void*, void*, void*,
+                               void*, void*, void*, void*, int, int, int, int,
+                               int, int, bool, bool, hipStream_t);
+hipError_t lfmq_moe_glu(const void*, const void*, const void*, const void*,
+                        const void*, void*, int, int, float, float, float,
+                        int, int, bool, hipStream_t);
+hipError_t lfmq_moe_down(const void*, const void*, const void*, void*, int,
+                         int, int, int, bool, hipStream_t);
+hipError_t lfmq_clamped_glu(const void*, void*, long, int, float, float,
+                            float, bool, hipStream_t);
 hipError_t lfmq_silu_mul_fused(const void*, void*, long, int, hipStream_t);
 hipError_t lfmq_silu_mul_any(const void*, void*, long, int, bool,
                              hipStream_t);
@@ -451,6 +494,309 @@ T_ attn_window_decode(T_ q, T_ ring, T_ seq, T_ cu, T_ slots, T_ lens,
   return part;
 }
 
+bool al16(const T_& t) { return ((u64)t.data_ptr() & 15) == 0; }
+
+// fp32 per-channel parameter of the given length
+const void* vec32(const T_& t, long n, const char* name) {
+  check(t, torch::kFloat32, name);
+  TORCH_CHECK(t.numel() == n, name, " must have ", n, " entries");
+  return t.data_ptr();
+}
+
+// {x, h}: x = rms(table[tok]) * w in fp32, h = x in the table's dtype (x
+// itself in 32 bit)
+std::vector<T_> embed_norm(T_ tok, T_ table, T_ w, double eps) {
+  check(tok, torch::kInt64, "tok");
+  const bool f32 = storage(table, "table");
+  check(table, table.scalar_type(), "table");
+  TORCH_CHECK(table.dim() == 2 && tok.numel() > 0, "embed_norm: shape");
+  const long n = tok.numel(), width = table.size(1);
+  const void* wp = vec32(w, width, "norm weight");
+  auto x = torch::empty({n, width}, table.options().dtype(torch::kFloat32));
+  T_ h = f32 ? x : torch::empty({n, width}, table.options());
+  CHECK_HIP(lfmq_embed_norm(x.data_ptr(), table.data_ptr(), tok.data_ptr(),
+                            wp, f32 ? nullptr : h.data_ptr(), (int)n,
+                            (int)width, (int)table.size(0), (float)eps, f32,
+                            stream()));
+  return {x, h};
+}
+
+struct NormOut {
+  T_ h;
+  const void* w_out;
+  void* hp;
+};
+
+NormOut norm_out(const T_& x, const OptT& w_out, bool f32) {
+  check(x, torch::kFloat32, "x");
+  TORCH_CHECK(x.dim() == 2 && x.size(0) > 0, "x must be [rows, width]");
+  NormOut o;
+  const bool copy = w_out.has_value() || !f32;
+  o.h = copy ? torch::empty_like(x, x.options().dtype(
+                                        f32 ? torch::kFloat32
+                                            : torch::kBFloat16))
+             : x;
+  o.hp = copy ? o.h.data_ptr() : nullptr;
+  o.w_out = w_out.has_value() ? vec32(*w_out, x.size(1), "output norm weight")
+                              : nullptr;
+  return o;
+}
+
+// x += rms(y) * w; returns x in y's dtype, or rms(x) * w_out * gain
+T_ post_norm(T_ x, T_ y, T_ w, double eps, OptT w_out, double gain) {
+  const bool f32 = storage(y, "y");
+  check(y, y.scalar_type(), "y");
+  const NormOut o = norm_out(x, w_out, f32);
+  TORCH_CHECK(y.sizes() == x.sizes(), "post_norm: shape mismatch");
+  CHECK_HIP(lfmq_post_norm(x.data_ptr(), y.data_ptr(),
+                           vec32(w, x.size(1), "norm weight"), o.w_out, o.hp,
+                           (int)x.size(0), (int)x.size(1), (float)eps,
+                           (float)gain, f32, stream()));
+  return o.h;
+}
+
+// the same, y the sum of rows[pos[t, :]] and sgate[t] * shared[t]
+T_ post_norm_experts(T_ x, T_ rows, T_ pos, OptT shared, OptT sgate, T_ w,
+                     double eps, OptT w_out, double gain) {
+  const bool f32 = storage(rows, "rows");
+  check(rows, rows.scalar_type(), "rows");
+  check(pos, torch::kInt32, "pos");
+  const NormOut o = norm_out(x, w_out, f32);
+  const long n = x.size(0), width = x.size(1);
+  TORCH_CHECK(rows.dim() == 2 && rows.size(1) == width && pos.dim() == 2 &&
+                  pos.size(0) == n && pos.numel() == rows.size(0),
+              "post_norm_experts: shape mismatch");
+  const void *sh = nullptr, *sg = nullptr;
+  if (shared.has_value()) {
+    check(*shared, rows.scalar_type(), "shared");
+    TORCH_CHECK(shared->numel() == n * width && sgate.has_value(),
+                "post_norm_experts: shared expert mismatch");
+    sh = shared->data_ptr();
+    sg = vec32(*sgate, n, "shared gate");
+  }
+  CHECK_HIP(lfmq_post_norm_experts(
+      x.data_ptr(), rows.data_ptr(), pos.data_ptr(), (int)pos.size(1), sh, sg,
+      vec32(w, width, "norm weight"), o.w_out, o.hp, (int)n, (int)width,
+      (float)eps, (float)gain, f32, stream()));
+  return o.h;
+}
+
+// in rows [q | k | v]; kc [slots, cap, kv, dim], vc [slots, cap, kv, dv]
+T_ qk_prep(T_ in, T_ seq, T_ cu, T_ slots, T_ lens, T_ wq, T_ wk, T_ inv_freq,
+           T_ kc, T_ vc, double eps) {
+  const SeqView sv = view(seq, cu, slots, lens);
+  const bool f32 = storage(in, "in");
+  check(kc, in.scalar_type(), "key cache");
+  check(vc, in.scalar_type(), "value cache");
+  check(wq, torch::kFloat32, "query norm");
+  check(inv_freq, torch::kFloat32, "inv_freq");
+  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == lens.numel() &&
+                  vc.size(0) == kc.size(0) && vc.size(1) == kc.size(1) &&
+                  vc.size(2) == kc.size(2),
+              "qk_prep: cache mismatch");
+  const long kv = kc.size(2), dim = kc.size(3), dv = vc.size(3);
+  const long nq = wq.numel(), nk = kv * dim, nv = kv * dv;
+  const long ld = row_stride(in, nq + nk + nv, "in"), half = inv_freq.numel();
+  TORCH_CHECK(in.size(0) == sv.n && nq > 0 && nq % dim == 0 &&
+                  2 * half <= dim,
+              "qk_prep: shape mismatch");
+  auto q = torch::empty({sv.n, nq}, in.options());
+  CHECK_HIP(lfmq_qk_prep(in.data_ptr(), ld, sv, wq.data_ptr(),
+                         vec32(wk, nk, "key norm"), inv_freq.data_ptr(),
+                         q.data_ptr(), kc.data_ptr(), vc.data_ptr(),
+                         (int)kc.size(1), (int)nq, (int)nk, (int)nv, (int)dim,
+                         (int)half, (float)eps, f32, stream()));
+  return q;
+}
+
+// q [N, heads * dim] ready, over the cache; writes out's columns
+void attn_grouped(T_ q, T_ kc, T_ vc, T_ seq, T_ cu, T_ slots, T_ lens,
+                  T_ sink, T_ out, double scale, double gain, long max_count,
+                  bool general) {
+  const SeqView sv = view(seq, cu, slots, lens);
+  const bool f32 = storage(q, "q");
+  check(q, q.scalar_type(), "q");
+  check(kc, q.scalar_type(), "key cache");
+  check(vc, q.scalar_type(), "value cache");
+  check(sink, torch::kFloat32, "sink");
+  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == lens.numel() &&
+                  vc.size(0) == kc.size(0) && vc.size(1) == kc.size(1) &&
+                  vc.size(2) == kc.size(2),
+              "attn_grouped: cache mismatch");
+  const long H = sink.numel(), kv = kc.size(2), dim = kc.size(3);
+  const long dv = vc.size(3), cap = kc.size(1);
+  const long ldo = row_stride(out, H * dv, "out");
+  TORCH_CHECK(H % kv == 0 && H <= 65535 && q.numel() == sv.n * H * dim &&
+                  out.size(0) == sv.n && out.scalar_type() == q.scalar_type(),
+              "attn_grouped: shape mismatch");
+  const int g = (int)(H / kv);
+  const bool fast = !f32 && !general &&
+                    lfmq_attn_grouped_mfma_ok(q.data_ptr(), kc.data_ptr(),
+                                              vc.data_ptr(), (int)dim,
+                                              (int)dv);
+  if (fast && max_count == 1 && sv.n == sv.b) {
+    const int splits = lfmq_attn_grouped_splits(sv.b, (int)H, g, (int)cap);
+    T_ part;
+    if (splits > 1)
+      part = torch::empty({sv.b, splits, H, dv + 2},
+                          q.options().dtype(torch::kFloat32));
+    CHECK_HIP(lfmq_attn_grouped_decode(
+        q.data_ptr(), kc.data_ptr(), vc.data_ptr(), sv, sink.data_ptr(),
+        splits > 1 ? part.data_ptr() : nullptr, out.data_ptr(), ldo, (int)H,
+        g, (int)dim, (int)dv, (int)cap, splits, (float)scale, (float)gain,
+        stream()));
+  } else if (fast) {
+    CHECK_HIP(lfmq_attn_grouped_mfma(
+        q.data_ptr(), kc.data_ptr(), vc.data_ptr(), sv, sink.data_ptr(),
+        out.data_ptr(), ldo, (int)H, g, (int)dim, (int)dv, (int)cap,
+        (float)scale, (float)gain, (int)max_count, stream()));
+  } else {
+    CHECK_HIP(lfmq_attn_grouped(q.data_ptr(), kc.data_ptr(), vc.data_ptr(),
+                                sv, sink.data_ptr(), out.data_ptr(), ldo,
+                                (int)H, g, (int)dim, (int)dv, (int)cap,
+                                (float)scale, (float)gain, f32, stream()));
+  }
+}
+
+// x and y: column views of one projection [N, *]; gw [blocks, 2, n, n],
+// gb [blocks, 2, n]; ring [slots, taps, C], S [slots, C].  tile0 [b] first
+// 64-token tile of each sequence, `tiles` in all.
+void gated_lru(T_ x, T_ y, T_ seq, T_ cu, T_ slots, T_ lens, T_ xb, T_ yb,
+               T_ cw, T_ cb, T_ gw, T_ gb, T_ lam, T_ ring, T_ S, T_ out,
+               double c, double gain, OptT tile0, long tiles, long max_count,
+               bool general) {
+  const SeqView sv = view(seq, cu, slots, lens);
+  const bool f32 = storage(x, "x");
+  check(gw, x.scalar_type(), "gate weights");
+  TORCH_CHECK(gw.dim() == 4 && gw.size(1) == 2 && gw.size(2) == gw.size(3),
+              "gate weights must be [blocks, 2, n, n]");
+  const long blocks = gw.size(0), n = gw.size(2), C = blocks * n;
+  const long ld = row_stride(x, C, "x"), ldo = row_stride(out, C, "out");
+  check(ring, torch::kFloat32, "conv ring");
+  check(S, torch::kFloat32, "S");
+  TORCH_CHECK(ring.dim() == 3 && ring.size(2) == C &&
+                  ring.size(0) == lens.numel() &&
+                  S.numel() == lens.numel() * C &&
+                  row_stride(y, C, "y") == ld && x.size(0) == sv.n &&
+                  y.size(0) == sv.n && out.size(0) == sv.n &&
+                  y.scalar_type() == x.scalar_type() &&
+                  out.scalar_type() == x.scalar_type() && blocks <= 65535,
+              "gated_lru: shape mismatch");
+  const long taps = ring.size(1);
+  const bool mfma =
+      !f32 && !general && lfmq_lru_mfma_ok(gw.data_ptr(), (int)n);
+  const bool single = sv.n == sv.b && max_count == 1;
+  T_ u, ab, ends;
+  if (!(mfma && single)) {
+    u = torch::empty({sv.n, C}, x.options());
+    ab = torch::empty({sv.n, C, 2}, S.options());
+  }
+  const void* t0 = nullptr;
+  if (mfma && !single) {
+    TORCH_CHECK(tile0.has_value() && tile0->numel() == sv.b && tiles >= sv.b,
+                "gated_lru: tiles missing");
+    check(*tile0, torch::kInt32, "tile0");
+    t0 = tile0->data_ptr();
+    ends = torch::empty({tiles, C, 2}, S.options());
+  }
+  auto ptr = [](const T_& t) { return t.defined() ? t.data_ptr() : nullptr; };
+  CHECK_HIP(lfmq_gated_lru(
+      sv, x.data_ptr(), y.data_ptr(), ld, vec32(xb, C, "x bias"),
+      vec32(yb, C, "y bias"), vec32(cw, C * taps, "conv weight"),
+      vec32(cb, C, "conv bias"), gw.data_ptr(), vec32(gb, 2 * C, "gate bias"),
+      vec32(lam, C, "lam"), ring.data_ptr(), S.data_ptr(), out.data_ptr(),
+      ldo, (int)C, (int)blocks, (int)taps, (float)c, (float)gain, ptr(u),
+      ptr(ab), ptr(ends), t0, (int)max_count, single, mfma, f32, stream()));
+}
+
+// rows a tile for `pairs` (token, choice) pairs; `aligned`: the matrix-core
+// products apply
+long moe_tile(long pairs, long experts, bool aligned) {
+  if (!aligned) return 8;
+  return pairs >= 32 * experts ? 128 : 16;
+}
+
+// w [E (+ 1 with the shared expert's gate), width].  Returns {src, weight,
+// pos [n, top], tiles [t, 3], shared gate [n] or empty}
+std::vector<T_> moe_route(T_ h, T_ w, long E, long top, long bm) {
+  const bool f32 = storage(h, "h");
+  check(h, h.scalar_type(), "h");
+  check(w, h.scalar_type(), "router");
+  const long n = h.size(0), width = h.size(1);
+  TORCH_CHECK(h.dim() == 2 && w.dim() == 2 && w.size(1) == width && n > 0 &&
+                  (w.size(0) == E || w.size(0) == E + 1) && top >= 1 &&
+                  top <= E && bm >= 1 && n * top < INT32_MAX,
+              "moe_route: shape mismatch");
+  const bool sg = w.size(0) > E;
+  const long pairs = n * top;
+  const long tiles = pairs / bm + (E < pairs ? E : pairs);
+  auto io = h.options().dtype(torch::kInt32);
+  auto fo = h.options().dtype(torch::kFloat32);
+  auto ids = torch::empty({pairs}, io), src = torch::empty({pairs}, io);
+  auto pos = torch::empty({n, top}, io), tl = torch::empty({tiles, 3}, io);
+  auto score = torch::empty({pairs}, fo), weight = torch::empty({pairs}, fo);
+  auto gate = torch::empty({sg ? n : 0}, fo);
+  const bool mfma = !f32 && width % 8 == 0 && al16(h) && al16(w);
+  CHECK_HIP(lfmq_moe_route_sort(
+      h.data_ptr(), w.data_ptr(), ids.data_ptr(), score.data_ptr(),
+      sg ? gate.data_ptr() : nullptr, src.data_ptr(), weight.data_ptr(),
+      pos.data_ptr(), tl.data_ptr(), (int)n, (int)width, (int)E, (int)top,
+      (int)bm, (int)tiles, mfma, f32, stream()));
+  return {src, weight, pos, tl, gate};
+}
+
+// act [pairs, ff] of h's rows src, gu [E, 2 ff, width]
+T_ moe_glu(T_ h, T_ gu, T_ src, T_ weight, T_ tiles, double limit,
+           double alpha, double beta, long bm) {
+  const bool f32 = storage(h, "h");
+  check(h, h.scalar_type(), "h");
+  check(gu, h.scalar_type(), "gate_up");
+  check(src, torch::kInt32, "src");
+  check(tiles, torch::kInt32, "tiles");
+  const long pairs = src.numel(), ff = gu.size(1) / 2, K = h.size(1);
+  TORCH_CHECK(gu.dim() == 3 && gu.size(2) == K && gu.size(1) == 2 * ff &&
+                  (bm < 16 || (!f32 && K % 8 == 0 && al16(h) && al16(gu))),
+              "moe_glu: shape mismatch");
+  auto out = torch::empty({pairs, ff}, h.options());
+  CHECK_HIP(lfmq_moe_glu(h.data_ptr(), gu.data_ptr(), src.data_ptr(),
+                         vec32(weight, pairs, "weight"), tiles.data_ptr(),
+                         out.data_ptr(), (int)ff, (int)K, (float)limit,
+                         (float)alpha, (float)beta, (int)tiles.size(0),
+                         (int)bm, f32, stream()));
+  return out;
+}
+
+// rows [pairs, width] of act [pairs, ff], down [E, width, ff]
+T_ moe_down(T_ act, T_ down, T_ tiles, long bm) {
+  const bool f32 = storage(act, "act");
+  check(act, act.scalar_type(), "act");
+  check(down, act.scalar_type(), "down");
+  check(tiles, torch::kInt32, "tiles");
+  const long K = act.size(1), N = down.size(1);
+  TORCH_CHECK(down.dim() == 3 && down.size(2) == K &&
+                  (bm < 16 || (!f32 && K % 8 == 0 && al16(act) && al16(down))),
+              "moe_down: shape mismatch");
+  auto out = torch::empty({act.size(0), N}, act.options());
+  CHECK_HIP(lfmq_moe_down(act.data_ptr(), down.data_ptr(), tiles.data_ptr(),
+                          out.data_ptr(), (int)N, (int)K, (int)tiles.size(0),
+                          (int)bm, f32, stream()));
+  return out;
+}
+
+T_ clamped_glu(T_ gu, double limit, double alpha, double beta) {
+  const bool f32 = storage(gu, "gate_up");
+  check(gu, gu.scalar_type(), "gate_up");
+  const long ff = gu.size(-1) / 2, rows = gu.numel() / gu.size(-1);
+  TORCH_CHECK(gu.size(-1) == 2 * ff && rows > 0, "odd gate_up width");
+  auto sizes = gu.sizes().vec();
+  sizes.back() = ff;
+  auto y = torch::empty(sizes, gu.options());
+  CHECK_HIP(lfmq_clamped_glu(gu.data_ptr(), y.data_ptr(), rows, (int)ff,
+                             (float)limit, (float)alpha, (float)beta, f32,
+                             stream()));
+  return y;
+}
+
 T_ silu_mul_fused(T_ gu) {
   const bool f32 = storage(gu, "gate_up");
   check(gu, gu.scalar_type(), "gate_up");
@@ -515,6 +861,18 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "windowed sink attention over a step's keys");
   m.def("attn_window_decode", &attn_window_decode,
         "windowed attention over the latent ring");
+  m.def("embed_norm", &embed_norm, "normed embedding rows");
+  m.def("post_norm", &post_norm, "norm a sublayer's output, add, cast or norm");
+  m.def("post_norm_experts", &post_norm_experts,
+        "sum of experts, normed, added, cast or normed");
+  m.def("qk_prep", &qk_prep, "query/key norms, rotation, cache write");
+  m.def("attn_grouped", &attn_grouped, "grouped-query sink attention");
+  m.def("gated_lru", &gated_lru, "convolution + gated linear recurrence");
+  m.def("moe_tile", &moe_tile, "rows a tile of the expert products");
+  m.def("moe_route", &moe_route, "sigmoid top-k router and expert sort");
+  m.def("moe_glu", &moe_glu, "gate/up products and clamped GLU");
+  m.def("moe_down", &moe_down, "down products of the experts");
+  m.def("clamped_glu", &clamped_glu, "clamped GLU on fused gate_up");
   m.def("silu_mul_fused", &silu_mul_fused, "silu-mul on fused gate_up");
   m.def("greedy_sample", &greedy_sample, "row argmax");
   m.def("advance_record", &advance_record, "graph decode-state advance");

@@ -154,8 +154,9 @@ def load(path: str, device: str = "cpu", tp_rank: int = 0, tp_world: int = 1,
         # assign=True would otherwise let the checkpoint dtype override an
         # explicitly requested one: cast float tensors here.
         keep = _fp32_names(model)
-        state = {k: (v.to(dtype) if v.is_floating_point() and k not in keep
-                     else v) for k, v in state.items()}
+        state = {k: (v.to(torch.float32 if k in keep else dtype)
+                     if v.is_floating_point() else v)
+                 for k, v in state.items()}
     model.load_state_dict(state, strict=True, assign=True)
     model = model.to(device)  # anything not in the checkpoint (none today)
     # assign=True unties tied embeddings (two independent tensors after the

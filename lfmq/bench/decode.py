@@ -41,6 +41,11 @@ def _bench_config(model_name: str, n_layers: Optional[int] = None):
         cfg = {"rapivik-1b": RapivikConfig.sized_1b,
                "rapivik-8b": RapivikConfig.sized_8b,
                "tiny-rapivik": RapivikConfig.tiny}[model_name]()
+    elif model_name in ("zatasun-1b", "zatasun-8b", "tiny-zatasun"):
+        from ..models.zatasun import ZatasunConfig
+        cfg = {"zatasun-1b": ZatasunConfig.sized_1b,
+               "zatasun-8b": ZatasunConfig.sized_8b,
+               "tiny-zatasun": ZatasunConfig.tiny}[model_name]()
     elif model_name == "tiny-debug":
         # contract-test shape only (tests/test_bench_contract.py);
         # never a reportable benchmark config

@@ -28,6 +28,9 @@ MODEL_PRESETS = {
     "rapivik-1b": ("rapivik", "sized_1b"),
     "rapivik-8b": ("rapivik", "sized_8b"),
     "tiny-rapivik": ("rapivik", "tiny"),
+    "zatasun-1b": ("zatasun", "sized_1b"),
+    "zatasun-8b": ("zatasun", "sized_8b"),
+    "tiny-zatasun": ("zatasun", "tiny"),
 }
 
 

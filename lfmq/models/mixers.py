@@ -8,12 +8,22 @@ interface, so that a model is a list of them:
                                  32 bits, computed inside the input norm
     forward(h, side, batch, cache, state) -> sublayer output [N, width]
 
-h [N, width] is the normed input in the model's dtype (bf16 or fp32).
+h [N, width] is the sublayer's input in the model's dtype (bf16 or fp32).
 Norm weights, gate biases and sinks are fp32 always.
+
+Mixers that can run side by side are written as branches of a
+ParallelMixer, which owns one input and one output projection for all:
+
+    rows_in, rows_out            columns of the input projection that the
+                                 branch reads, and of its result
+    state_spec(max_seq)          as above
+    mix(p, out, gain, batch, cache, state)
+                                 p [N, rows_in] -> out [N, rows_out], both
+                                 column views; the result is times gain
 """
 from __future__ import annotations
 
-from typing import Optional
+from typing import Dict, NamedTuple, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -153,6 +163,114 @@ class LatentAttention(nn.Module):
         return self.o_proj(o)
 
 
+class GroupedAttention(nn.Module):
+    """Branch: causal grouped-query attention with RMS norms over the whole
+    query and key projections, rotary positions and a softmax sink per head.
+    The cache keeps keys (normed and rotated) and values of every token.
+    rot_scaling: the wavelength-dependent frequency scaling of
+    lfmq.ops.functional.rope_inv_freq."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int,
+                 scale: float, rot_dims: int, rot_base: float,
+                 rot_scaling: Optional[dict], eps: float, dtype):
+        super().__init__()
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError(f"cannot rotate {rot_dims} of {dim} dimensions")
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads do not share {kv_heads}")
+        self.kv_heads, self.dim, self.vdim = kv_heads, dim, vdim
+        self.scale, self.eps, self.dtype = scale, eps, dtype
+        self.rot = (rot_dims, rot_base, rot_scaling)
+        # [queries | keys | values]
+        self.rows_in = heads * dim + kv_heads * (dim + vdim)
+        self.rows_out = heads * vdim
+        self.q_norm = _fp32(heads * dim, 1.0)
+        self.k_norm = _fp32(kv_heads * dim, 1.0)
+        self.sink = _fp32(heads)
+
+    def state_spec(self, max_seq: int) -> dict:
+        # rows of later positions are written before they are read
+        return {n: ((max_seq, self.kv_heads, d), self.dtype, "by_position")
+                for n, d in (("k", self.dim), ("v", self.vdim))}
+
+    def mix(self, p, out, gain, batch, cache, state):
+        dims, base, scaling = self.rot
+        inv = F.rope_inv_freq(dims, base, p.device, scaling)
+        q = F.qk_prep(p, batch, cache, self.q_norm, self.k_norm, inv,
+                      state["k"], state["v"], self.eps)
+        F.attn_grouped(q, state["k"], state["v"], batch, cache, self.sink,
+                       out, self.scale, gain)
+
+
+class GatedLRU(nn.Module):
+    """Branch: a real-gated linear recurrent unit behind a short causal
+    convolution, times a gelu branch.  Both gates of the recurrence are
+    block-diagonal; decay = exp(decay_c * r * softplus(lam))."""
+
+    decay_c = -8.0
+
+    def __init__(self, width: int, blocks: int, taps: int, dtype):
+        super().__init__()
+        if width % blocks:
+            raise ValueError(f"{blocks} blocks do not divide width {width}")
+        n = width // blocks
+        self.width, self.taps = width, taps
+        self.rows_in, self.rows_out = 2 * width, width    # [gelu | conv]
+        self.y_b, self.x_b = _fp32(width), _fp32(width)
+        self.conv_w = nn.Parameter(torch.zeros(width, taps))
+        self.conv_b = _fp32(width)
+        # [recurrence gate | input gate] of every block, [out, in]
+        self.gate_w = nn.Parameter(torch.zeros(blocks, 2, n, n, dtype=dtype))
+        self.gate_b = nn.Parameter(torch.zeros(blocks, 2, n))
+        self.lam = _fp32(width)
+
+    def state_spec(self, max_seq: int) -> dict:
+        return {"S": ((self.width,), torch.float32),
+                "conv": ((self.taps, self.width), torch.float32)}
+
+    def mix(self, p, out, gain, batch, cache, state):
+        F.gated_lru(p[:, self.width:], p[:, :self.width], batch, cache,
+                    self.x_b, self.y_b, self.conv_w, self.conv_b, self.gate_w,
+                    self.gate_b, self.lam, state["conv"], state["S"], out,
+                    self.decay_c, gain)
+
+
+class ParallelMixer(nn.Module):
+    """Branches side by side on one input: one projection in, one out, the
+    sum of the branches' outputs weighted by their gains."""
+
+    def __init__(self, width: int, branches: Dict[str, Tuple[nn.Module, float]],
+                 dtype):
+        super().__init__()
+        self.branches = nn.ModuleDict({k: b for k, (b, _) in branches.items()})
+        self.gains = {k: g for k, (_, g) in branches.items()}
+        bs = self.branches.values()
+        self.rows_in = sum(b.rows_in for b in bs)
+        self.rows_out = sum(b.rows_out for b in bs)
+        self.in_proj = nn.Linear(width, self.rows_in, bias=False, dtype=dtype)
+        self.o_proj = nn.Linear(self.rows_out, width, bias=False, dtype=dtype)
+
+    def state_spec(self, max_seq: int) -> dict:
+        return {f"{n}.{k}": v for n, b in self.branches.items()
+                for k, v in b.state_spec(max_seq).items()}
+
+    def side(self):
+        return None, None
+
+    def forward(self, h, side, batch, cache, state):
+        p = self.in_proj(h)
+        out = torch.empty(p.shape[0], self.rows_out, dtype=p.dtype,
+                          device=p.device)
+        i = o = 0
+        for n, b in self.branches.items():
+            b.mix(p[:, i:i + b.rows_in], out[:, o:o + b.rows_out],
+                  self.gains[n], batch, cache,
+                  {k[len(n) + 1:]: t for k, t in state.items()
+                   if k.startswith(n + ".")})
+            i, o = i + b.rows_in, o + b.rows_out
+        return self.o_proj(out)
+
+
 class DenseMLP(nn.Module):
     """down(silu(gate h) * up h), gate and up fused."""
 
@@ -164,6 +282,99 @@ class DenseMLP(nn.Module):
 
     def forward(self, h):
         return self.down_proj(F.silu_mul_gateup(self.gate_up_proj(h), self.ff))
+
+
+class ExpertSum(NamedTuple):
+    """A feed-forward's output not yet summed: token t's is the sum of
+    rows[pos[t, :]] and, with a shared expert, sgate[t] * shared[t]."""
+    rows: torch.Tensor
+    pos: torch.Tensor
+    shared: Optional[torch.Tensor]
+    sgate: Optional[torch.Tensor]
+
+
+class ClampedGLU(nn.Module):
+    """down(g sigmoid(alpha g) (u + beta)), g = min(gate h, limit) and
+    u = clamp(up h, -limit, limit)."""
+
+    def __init__(self, width: int, ff: int, limit: float, alpha: float,
+                 beta: float, dtype):
+        super().__init__()
+        self.act = (limit, alpha, beta)
+        self.gate_up_proj = nn.Linear(width, 2 * ff, bias=False, dtype=dtype)
+        self.down_proj = nn.Linear(ff, width, bias=False, dtype=dtype)
+
+    def forward(self, h):
+        return self.down_proj(F.clamped_glu(self.gate_up_proj(h), *self.act))
+
+
+class ExpertMLP(nn.Module):
+    """Mixture of clamped-GLU experts.  A token goes to the `top` experts
+    with the largest sigmoid scores; the score (not renormalized) weights
+    the expert's input.  A shared expert runs for every token, times the
+    sigmoid of one output of its own.  Returns an ExpertSum."""
+
+    def __init__(self, width: int, experts: int, top: int, ff: int,
+                 limit: float, alpha: float, beta: float,
+                 shared: Optional[ClampedGLU], dtype):
+        super().__init__()
+        if not 1 <= top <= experts:
+            raise ValueError(f"cannot choose {top} of {experts} experts")
+        self.experts, self.top = experts, top
+        self.act = (limit, alpha, beta)
+        # a router row per expert, then the shared expert's gate
+        self.router = nn.Parameter(torch.zeros(
+            experts + (shared is not None), width, dtype=dtype))
+        self.gate_up = nn.Parameter(torch.zeros(experts, 2 * ff, width,
+                                                dtype=dtype))
+        self.down = nn.Parameter(torch.zeros(experts, width, ff, dtype=dtype))
+        self.shared = shared
+
+    def forward(self, h) -> ExpertSum:
+        rows, pos, sgate = F.moe(h, self.router, self.gate_up, self.down,
+                                 self.top, self.act)
+        if self.shared is None:
+            return ExpertSum(rows, pos, None, None)
+        return ExpertSum(rows, pos, self.shared(h), sgate)
+
+
+class PostNorm(nn.Module):
+    """RMS norm on a sublayer's output, added to the fp32 residual stream."""
+
+    def __init__(self, dim: int, eps: float):
+        super().__init__()
+        self.weight, self.eps = _fp32(dim, 1.0), eps
+
+    def forward(self, x, y, out: Optional[nn.Module] = None,
+                gain: float = 1.0):
+        """x += norm(y) in place; returns x in y's dtype, or out's norm of
+        it times gain."""
+        w_out = None if out is None else out.weight
+        if isinstance(y, ExpertSum):
+            return F.post_norm_experts(x, y, self.weight, self.eps, w_out,
+                                       gain)
+        return F.post_norm(x, y, self.weight, self.eps, w_out, gain)
+
+
+class PostNormBlock(nn.Module):
+    """Block whose norms sit on the sublayers' outputs: the sublayers read
+    the fp32 residual x itself (h: x in the model's dtype).  Returns the
+    next h; last: (the model's output norm, gain) behind the last block."""
+
+    def __init__(self, mixer: nn.Module, mlp: Optional[nn.Module], width: int,
+                 eps: float):
+        super().__init__()
+        self.mixer = mixer
+        self.norm1 = PostNorm(width, eps)
+        if mlp is not None:
+            self.norm2 = PostNorm(width, eps)
+        self.mlp = mlp
+
+    def forward(self, x, h, batch, cache, state, last=(None, 1.0)):
+        y = self.mixer(h, None, batch, cache, state)
+        if self.mlp is None:
+            return self.norm1(x, y, *last)
+        return self.norm2(x, self.mlp(self.norm1(x, y)), *last)
 
 
 class MixerBlock(nn.Module):

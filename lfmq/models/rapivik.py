@@ -10,7 +10,7 @@ from __future__ import annotations
 
 import copy
 from dataclasses import dataclass
-from typing import Dict, List, Optional, Sequence
+from typing import Dict, List
 
 import torch
 import torch.nn as nn
@@ -18,6 +18,7 @@ import torch.nn as nn
 from ..ops import functional as F
 from .mixers import (DenseMLP, LatentAttention, MixerBlock, MLSTMMixer,
                      ResidualNorm)
+from .packed import PackedCausalLM
 from .seqcache import SequenceCache, StepBatch
 
 MIXER_TYPES = ("mlstm", "latent_attention")
@@ -139,12 +140,9 @@ def _make_mixer(e: dict, width: int, eps: float, dtype) -> nn.Module:
                            m["rot"]["dims"], eps, dtype)
 
 
-class RapivikForCausalLM(nn.Module):
-    packed = True            # takes unequal sequences in one batch
-
+class RapivikForCausalLM(PackedCausalLM):
     def __init__(self, cfg: RapivikConfig, dtype=torch.bfloat16):
-        super().__init__()
-        self.cfg, self.dtype = cfg, dtype
+        super().__init__(cfg, dtype)
         w, eps = cfg.hidden_size, cfg.rms_eps
         self.embed_tokens = nn.Embedding(cfg.vocab_size, w, dtype=dtype)
         # one row per bucket, and one for "no previous token"
@@ -160,33 +158,11 @@ class RapivikForCausalLM(nn.Module):
         self.norm = ResidualNorm(w, eps, True, dtype)
         self.lm_head = nn.Linear(w, cfg.vocab_size, bias=False, dtype=dtype)
 
-    def fp32_names(self) -> set:
-        """Parameters that keep 32 bits whatever the model's dtype."""
-        return {n for n, p in self.named_parameters()
-                if p.dim() == 1 and p.dtype == torch.float32}
+    def layer_mixers(self) -> list:
+        return [self.blocks[b].mixer for b in self.order]
 
-    @torch.no_grad()
-    def init_random(self, seed: int = 0):
-        g = torch.Generator().manual_seed(seed)
-        for p in self.parameters():
-            t = torch.randn(p.shape, generator=g, dtype=torch.float32) * 0.02
-            # 1-D parameters start at what they stand for (0 or 1)
-            p.data.copy_((p.data.float().cpu() + t if p.dim() == 1 else t)
-                         .to(p.dtype))
-        return self
-
-    def make_cache(self, batch: int, max_seq: Optional[int] = None,
-                   device=None) -> SequenceCache:
-        dev = device or self.norm.weight.device
-        max_seq = max_seq or self.cfg.max_seq
-        specs = [self.blocks[b].mixer.state_spec(max_seq) for b in self.order]
-        return SequenceCache(specs, batch, max_seq, dev)
-
-    # ---- the step function ----------------------------------------------
     def _run(self, tokens: torch.Tensor, batch: StepBatch,
              cache: SequenceCache, select=None, trace=None) -> torch.Tensor:
-        if not tokens.is_cuda:
-            raise RuntimeError("Rapivik runs on a GPU device only")
         x = F.bigram_embed(tokens, batch, cache, self.embed_tokens.weight,
                            self.bigram.weight, self.cfg.bigram["mul_prev"],
                            self.cfg.bigram["mul_cur"])
@@ -201,48 +177,6 @@ class RapivikForCausalLM(nn.Module):
             if h.shape[0] == 0:
                 return h.new_empty(0, self.cfg.vocab_size)
         return self.lm_head(h)
-
-    def forward_tokens(self, tokens: torch.Tensor, batch: StepBatch,
-                       cache: SequenceCache, select=None,
-                       trace: Optional[list] = None) -> torch.Tensor:
-        """One step of packed sequences: tokens [N] -> logits of all rows,
-        or of the `select`ed ones (int64 row numbers).  Advances the cache.
-        trace collects the residual stream after every layer run."""
-        logits = self._run(tokens, batch, cache, select, trace)
-        cache.advance(tokens, batch)
-        return logits
-
-    def forward(self, input_ids: torch.Tensor, cache: SequenceCache,
-                lengths: Optional[Sequence[int]] = None) -> torch.Tensor:
-        """input_ids [b, s] on slots 0..b-1 -> logits [b, s, vocab].  With
-        lengths, row i brings its first lengths[i] tokens and the result is
-        the last one's logits, [b, 1, vocab]."""
-        b, s = input_ids.shape
-        if lengths is None:
-            batch = cache.batch(range(b), [s] * b)
-            return self.forward_tokens(input_ids.reshape(-1).contiguous(),
-                                       batch, cache).view(b, s, -1)
-        batch = cache.batch(range(b), lengths)
-        tok = torch.cat([input_ids[i, :n] for i, n in enumerate(lengths)])
-        last = torch.tensor(batch.last_rows_host, device=tok.device)
-        return self.forward_tokens(tok, batch, cache, last).unsqueeze(1)
-
-    def forward_decode_step(self, input_ids, cache, state, max_seq):
-        """hipGraph-capturable: [b, 1] ids -> [b, 1, vocab].  Positions come
-        from the cache's own device lengths (state and max_seq belong to
-        the scalar-position models)."""
-        batch = cache.decode_batch(input_ids.shape[0])
-        tok = input_ids.reshape(-1).contiguous()
-        logits = self._run(tok, batch, cache)
-        F.seq_advance(tok, batch, cache)
-        return logits.unsqueeze(1)
-
-    @torch.no_grad()
-    def generate(self, input_ids, max_new_tokens: int = 32, cache=None,
-                 gen_cfg=None, generator=None):
-        from .generation import autoregressive_generate
-        return autoregressive_generate(self, input_ids, max_new_tokens,
-                                       cache, gen_cfg, generator)
 
 
 # ---------------------------------------------------------------------------

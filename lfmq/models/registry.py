@@ -13,10 +13,10 @@ from typing import Callable, Optional
 
 import torch
 
+from . import rapivik, zatasun
 from .llama import LlamaConfig, LlamaForCausalLM
 from .mixtral import MixtralConfig, MixtralForCausalLM
 from .opt import OPTConfig, OPTForCausalLM
-from .rapivik import RapivikConfig, RapivikForCausalLM, convert_state
 
 
 @dataclass(frozen=True)
@@ -32,8 +32,10 @@ ARCHS = {
     "llama": ArchSpec(LlamaConfig, LlamaForCausalLM, torch.bfloat16),
     "opt": ArchSpec(OPTConfig, OPTForCausalLM, torch.float32),
     "mixtral": ArchSpec(MixtralConfig, MixtralForCausalLM, torch.bfloat16),
-    "rapivik": ArchSpec(RapivikConfig, RapivikForCausalLM, torch.bfloat16,
-                        convert_state),
+    "rapivik": ArchSpec(rapivik.RapivikConfig, rapivik.RapivikForCausalLM,
+                        torch.bfloat16, rapivik.convert_state),
+    "zatasun": ArchSpec(zatasun.ZatasunConfig, zatasun.ZatasunForCausalLM,
+                        torch.bfloat16, zatasun.convert_state),
 }
 
 

@@ -3,7 +3,7 @@
 A SequenceCache has `n_slots` slots; a slot holds everything one live
 sequence carries from step to step: its length, its previous token, and
 what each layer run declares through its mixer's `state_spec` (a ring of
-latent rows, a recurrent matrix, ...).  Slots are handed out and given
+latent rows, keys and values, a recurrent state, ...).  Slots are handed out and given
 back; a slot of length 0 is fresh whatever its tensors hold, so giving one
 back costs no clearing pass.
 
@@ -40,6 +40,7 @@ class StepBatch:
             cu.append(cu[-1] + c)
             seq += [i] * c
         self.single = self.n == self.b          # one token each
+        self.max_count = max(counts)
         self.last_rows_host = [c - 1 for c in cu[1:]]
         t = self._dev(seq + cu + self.slot_ids)
         self.seq = t[:self.n]
@@ -72,7 +73,6 @@ class StepBatch:
             self._rows[window] = r
         return r
 
-
     def chunks(self, size: int):
         """(first chunk of every sequence, chunks in all) when sequences
         are cut into chunks of `size` tokens."""
@@ -87,7 +87,9 @@ class StepBatch:
 
 class SequenceCache:
     def __init__(self, specs: List[dict], n_slots: int, max_seq: int, device):
-        """specs: per layer run, name -> (shape per slot, dtype)."""
+        """specs: per layer run, name -> (shape per slot, dtype) and, for
+        rows that a position owns and writes before anyone reads them,
+        "by_position": nothing of theirs has to be kept apart."""
         self.specs, self.max_seq = specs, max_seq
         self.device = torch.device(device)
         self.n_slots = n_slots
@@ -97,7 +99,8 @@ class SequenceCache:
         self.turn = torch.zeros(n_slots, **i32)
         self.layers = [{k: torch.zeros((n_slots, *shape), dtype=dt,
                                        device=self.device)
-                        for k, (shape, dt) in spec.items()} for spec in specs]
+                        for k, (shape, dt, *_) in spec.items()}
+                       for spec in specs]
         self.lens_host = [0] * n_slots
         self._free = list(range(n_slots - 1, -1, -1))
         self._decode: Dict[int, StepBatch] = {}
@@ -182,13 +185,15 @@ class SequenceCache:
     def snapshot(self):
         """Everything a warm-up step would change."""
         return ([t.clone() for t in (self.lens, self.prev, self.turn)],
-                [{k: t.clone() for k, t in st.items()} for st in self.layers],
+                [{k: t.clone() for k, t in st.items()
+                  if "by_position" not in spec[k][2:]}
+                 for spec, st in zip(self.specs, self.layers)],
                 list(self.lens_host))
 
     def restore(self, snap) -> None:
         for t, old in zip((self.lens, self.prev, self.turn), snap[0]):
             t.copy_(old)
         for st, old in zip(self.layers, snap[1]):
-            for k in st:
+            for k in old:
                 st[k].copy_(old[k])
         self.lens_host = list(snap[2])

@@ -304,13 +304,31 @@ def head_norm_gate(o, gate, weight, eps: float) -> torch.Tensor:
                   "head_norm_gate")
 
 
-def rope_inv_freq(dims: int, base: float, device) -> torch.Tensor:
-    """fp32 base^(-2i/dims), i < dims/2, from a double-precision power."""
-    key = ("f64", dims, float(base), str(device))
+def _scaled_freq(f: float, factor: float, low: float, high: float,
+                 original: float) -> float:
+    """Context extension by wavelength: short waves keep their frequency,
+    long ones are slowed by `factor`, those between are blended."""
+    turns = original * f / (2 * math.pi)     # within the original context
+    if turns < low:
+        return f / factor
+    if turns > high:
+        return f
+    s = (turns - low) / (high - low)
+    return (1 - s) * f / factor + s * f
+
+
+def rope_inv_freq(dims: int, base: float, device,
+                  scaling: Optional[dict] = None) -> torch.Tensor:
+    """fp32 base^(-2i/dims), i < dims/2, computed in double precision.
+    scaling: {factor, low, high, original} of _scaled_freq."""
+    key = ("f64", dims, float(base), str(device),
+           tuple(sorted(scaling.items())) if scaling else None)
     t = _INV_FREQ_CACHE.get(key)
     if t is None:
-        i = torch.arange(dims // 2, dtype=torch.float64)
-        t = (float(base) ** (-2.0 * i / dims)).float().to(device)
+        f = [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)]
+        if scaling:
+            f = [_scaled_freq(x, **scaling) for x in f]
+        t = torch.tensor(f, dtype=torch.float64).float().to(device)
         _INV_FREQ_CACHE[key] = t
     return t
 
@@ -358,3 +376,75 @@ def attn_window_decode(q, ring, batch, cache, rank: int, window: int,
     splits = max(1, min(-(-reach // 64), -(-512 // groups), 64))
     return seq_ext().attn_window_decode(q, ring, *batch.view(cache), rank,
                                         window, splits, scale, general)
+
+
+def embed_norm(tokens, table, weight, eps: float):
+    """(x, h): normed embedding rows as the fp32 residual, and in the
+    table's dtype."""
+    return seq_ext().embed_norm(tokens, table, weight, eps)
+
+
+def post_norm(x, y, weight, eps: float, w_out=None, gain: float = 1.0):
+    """x += rms_norm(y) * weight in place (fp32 residual).  Returns x in y's
+    dtype (x itself in 32 bit) or, given w_out, rms_norm(x) * w_out * gain."""
+    return _guard(seq_ext().post_norm(x, y, weight, eps, w_out, gain),
+                  "post_norm")
+
+
+def post_norm_experts(x, y, weight, eps: float, w_out=None,
+                      gain: float = 1.0):
+    """post_norm of a lfmq.models.mixers.ExpertSum."""
+    return _guard(seq_ext().post_norm_experts(
+        x, y.rows, y.pos, y.shared, y.sgate, weight, eps, w_out, gain),
+        "post_norm_experts")
+
+
+def qk_prep(proj, batch, cache, q_norm, k_norm, inv_freq, kc, vc,
+            eps: float) -> torch.Tensor:
+    """[q | k | v] columns: norms over all of q and all of k, rotation; keys
+    and values go to the cache, queries [N, heads * dim] are returned."""
+    return seq_ext().qk_prep(proj, *batch.view(cache), q_norm, k_norm,
+                             inv_freq, kc, vc, eps)
+
+
+def attn_grouped(q, kc, vc, batch, cache, sink, out, scale: float,
+                 gain: float = 1.0, general: bool = False) -> None:
+    """Causal grouped-query attention with a sink over the cache, written to
+    out's columns.  general: the any-size kernel also where a matrix-core
+    one applies."""
+    seq_ext().attn_grouped(q, kc, vc, *batch.view(cache), sink, out, scale,
+                           gain, batch.max_count, general)
+    _guard(out, "attn_grouped")
+
+
+LRU_TILE = 64            # tokens a tile of the prompt kernels
+
+
+def gated_lru(x, y, batch, cache, x_b, y_b, conv_w, conv_b, gate_w, gate_b,
+              lam, ring, S, out, c: float, gain: float = 1.0,
+              general: bool = False) -> None:
+    """Convolution, gates, linear recurrence and gelu branch over the step's
+    rows (csrc/gated_lru.hip), written to out's columns."""
+    base, total = (None, 0) if batch.single else batch.chunks(LRU_TILE)
+    seq_ext().gated_lru(x, y, *batch.view(cache), x_b, y_b, conv_w, conv_b,
+                        gate_w, gate_b, lam, ring, S, out, c, gain, base,
+                        total, batch.max_count, general)
+    _guard(out, "gated_lru")
+
+
+def clamped_glu(gate_up, limit: float, alpha: float, beta: float):
+    return seq_ext().clamped_glu(gate_up, limit, alpha, beta)
+
+
+def moe(h, router, gate_up, down, top: int, act, general: bool = False):
+    """Router, sort by expert and expert products: (rows [N * top, width],
+    pos [N, top] row of a token's choice, the shared expert's gate [N] if
+    the router has its row).  Stays on the device."""
+    ext = seq_ext()
+    E, ff2, width = gate_up.shape
+    aligned = not general and h.dtype == torch.bfloat16 and \
+        width % 8 == 0 and ff2 % 16 == 0
+    bm = ext.moe_tile(h.shape[0] * top, E, aligned)
+    src, weight, pos, tiles, sgate = ext.moe_route(h, router, E, top, bm)
+    a = ext.moe_glu(h, gate_up, src, weight, tiles, *act, bm)
+    return _guard(ext.moe_down(a, down, tiles, bm), "moe"), pos, sgate

@@ -3,8 +3,8 @@
     PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace
 
   lfmq_hip  weight-quantized Llama / Mixtral / OPT kernels
-  lfmq_seq  recurrent and latent-attention layers, packed batches, and the
-            small ops that every model uses
+  lfmq_seq  recurrent, attention and expert layers on packed batches, and
+            the small ops that every model uses
 
 LFMQ_EXTENSIONS=lfmq_seq builds only the named ones (comma-separated).
 The built .so files land at the repo root, next to the package.
@@ -53,6 +53,11 @@ SEQ_SOURCES = [
     "csrc/attn_window.hip",
     "csrc/attn_window_mfma.hip",
     "csrc/attn_latent_mfma.hip",
+    "csrc/attn_grouped_decode.hip",
+    "csrc/qk_prep.hip",
+    "csrc/gated_lru.hip",
+    "csrc/moe_experts.hip",
+    "csrc/post_norm.hip",
     "csrc/elementwise.hip",
     "csrc/sample.hip",
 ]
