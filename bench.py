@@ -42,9 +42,11 @@ def main():
     ap.add_argument("--no-fidelity", action="store_true",
                     help="skip the delta-ppl/logit-KL fidelity pass")
     ap.add_argument("--compare", default="", metavar="SIZE",
-                    help="instead: prefill and decode throughput of Rapivik "
-                         "beside Llama at equal sizes (2k, 4k), one JSON "
-                         "line per shape")
+                    help="instead: prefill and decode throughput of the "
+                         "--models side by side at equal sizes (2k, 4k), one "
+                         "JSON line per shape")
+    ap.add_argument("--models", default="llama,rapivik", metavar="A,B,..",
+                    help="with --compare: llama, rapivik, zatasun")
     ap.add_argument("--phase", default="", choices=["", "prefill", "decode"],
                     help="with --compare: only this phase")
     ap.add_argument("--shape", default="", metavar="BATCHxLENGTH",
@@ -59,6 +61,7 @@ def main():
             b, n = map(int, args.shape.split("x"))
             pre = dec = ((b, n),)
         for row in compare(args.compare, args.layers or 8,
+                           tuple(args.models.split(",")),
                            prefill=() if args.phase == "decode" else pre,
                            decode=() if args.phase == "prefill" else dec):
             print(json.dumps(row), flush=True)

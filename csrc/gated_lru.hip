@@ -24,28 +24,54 @@ constexpr int SKC = 512;    // the same, single tokens
 struct LruArgs {
   const void *x, *y;        // projection columns, row stride ld
   u64 ld;
-  const float *xb, *yb, *cw, *cb, *gb, *lam;   // cw [C, taps], gb [B, 2, n]
+  const float *xb, *yb, *cw, *cb, *gb, *lam;   // cw [taps, C], gb [B, 2, n]
   const void* gw;           // [B, 2, n, n] rows = outputs
   float *ring, *S;
   void* out;
   u64 ldo;
   int C, blocks, n, taps;
   float c, gain;
+  bool x4;                  // four columns of x may be loaded at once
 };
 
 __device__ __forceinline__ float softplus_f(float x) {
   return x > 20.f ? x : log1pf(expf(x));
 }
+// FAST: the hardware's exponential, reciprocal and root, each good to a few
+// units in the last place (32-bit storage takes the library's)
+template <bool FAST>
+__device__ __forceinline__ float sigm(float x) {
+  if constexpr (FAST) return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+  return sigmoid_f(x);
+}
+// 0.5 x (1 + tanh(t)) = x sigmoid(2 t)
+template <bool FAST>
 __device__ __forceinline__ float gelu_tanh_f(float x) {
   const float k = 0.7978845608028654f;
-  return 0.5f * x * (1.f + tanhf(k * fmaf(0.044715f * x * x, x, x)));
+  return x * sigm<FAST>(2.f * k * fmaf(0.044715f * x * x, x, x));
 }
-// gate pre-activations and u -> decay and input
+// gate pre-activations and u -> decay and input.  1 - a^2 = -(e^t - 1) with
+// t = 2 log a, by its series where the difference would cancel.
+template <bool FAST>
 __device__ __forceinline__ void lru_pair(float r, float i, float u, float csp,
                                          float& a, float& z) {
-  const float la = csp * sigmoid_f(r);
-  a = expf(la);
-  z = sqrtf(-expm1f(2.f * la)) * sigmoid_f(i) * u;
+  const float la = csp * sigm<FAST>(r);
+  if constexpr (FAST) {
+    a = __expf(la);
+    const float t = 2.f * la;
+    float s = 1.f + t * (1.f / 8.f);
+    s = fmaf(t * (1.f / 7.f), s, 1.f);
+    s = fmaf(t * (1.f / 6.f), s, 1.f);
+    s = fmaf(t * (1.f / 5.f), s, 1.f);
+    s = fmaf(t * (1.f / 4.f), s, 1.f);
+    s = fmaf(t * (1.f / 3.f), s, 1.f);
+    s = fmaf(t * (1.f / 2.f), s, 1.f);
+    const float d = t > -0.5f ? -t * s : fmaf(-a, a, 1.f);
+    z = __builtin_amdgcn_sqrtf(d) * sigm<true>(i) * u;
+  } else {
+    a = expf(la);
+    z = sqrtf(-expm1f(2.f * la)) * sigm<false>(i) * u;
+  }
 }
 __device__ __forceinline__ float round_to(float v, const float*) { return v; }
 __device__ __forceinline__ float round_to(float v, const bf16_t*) {
@@ -66,56 +92,79 @@ __device__ __forceinline__ float conv_at(const LruArgs& A, int row, int row0,
                                          int pos, int slot, int c) {
   float v = A.cb[c];
   for (int j = 0; j < A.taps; ++j)
-    v = fmaf(A.cw[(u64)c * A.taps + j],
+    v = fmaf(A.cw[(u64)j * A.C + c],
              conv_in<T>(A, row, row0, pos, slot, A.taps - 1 - j, c), v);
   return round_to(v, (const T*)nullptr);
 }
 
-// u [n, C]; a thread takes one channel of RC consecutive rows and keeps the
-// last inputs in registers when there are four taps
-constexpr int RC = 8;
+template <typename T>
+__device__ __forceinline__ void load_x4(const LruArgs& A, int row, int c,
+                                        float v[4]) {
+  const T* p = (const T*)A.x + (u64)row * A.ld + c;
+  if (A.x4) {
+    ldf4(p, v);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = ldf(p + e);
+  }
+}
+
+constexpr int RC = 8;       // consecutive rows of a thread
+
+// u [n, C].  Four taps and C % 4 == 0: a thread takes four channels and
+// keeps the last inputs in registers
+template <typename T>
+__global__ __launch_bounds__(256) void lru_conv4_kernel(SeqView sv, LruArgs A,
+                                                        T* __restrict__ u) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  if (c >= A.C) return;
+  const int r0 = blockIdx.y * RC, r1 = min(r0 + RC, sv.n);
+  float w[4][4], in[4][4] = {}, b[4], xb[4], nx[RC][4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) ldf4(A.cw + (u64)j * A.C + c, w[j]);
+  ldf4(A.cb + c, b);
+  ldf4(A.xb + c, xb);
+#pragma unroll
+  for (int i = 0; i < RC; ++i)
+    if (r0 + i < r1) load_x4<T>(A, r0 + i, c, nx[i]);
+  int last = -1;
+#pragma unroll
+  for (int i = 0; i < RC; ++i) {
+    const int row = r0 + i;
+    if (row >= r1) break;
+    const int s = sv.seq[row];
+    if (s != last) {        // the three inputs before this one
+      const int slot = sv.slots[s], row0 = sv.cu[s];
+      const int pos = sv.lens[slot] + row - row0;
+#pragma unroll
+      for (int j = 1; j < 4; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          in[4 - j][e] = conv_in<T>(A, row, row0, pos, slot, j, c + e);
+      last = s;
+    }
+    float v[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      in[0][e] = in[1][e];
+      in[1][e] = in[2][e];
+      in[2][e] = in[3][e];
+      in[3][e] = nx[i][e] + xb[e];
+      v[e] = b[e];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[e] = fmaf(w[j][e], in[j][e], v[e]);
+    }
+    stf4(u + (u64)row * A.C + c, v);
+  }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void lru_conv_kernel(SeqView sv, LruArgs A,
                                                        T* __restrict__ u) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= A.C) return;
-  const int r0 = blockIdx.y * RC, r1 = min(r0 + RC, sv.n);
-  if (A.taps == 4) {
-    float w[4], in[4] = {}, b = A.cb[c], xb = A.xb[c];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) w[j] = A.cw[(u64)c * 4 + j];
-    float nx[RC];
-#pragma unroll
-    for (int i = 0; i < RC; ++i)
-      nx[i] = r0 + i < r1 ? ldf((const T*)A.x + (u64)(r0 + i) * A.ld + c) + xb
-                          : 0.f;
-    int last = -1;
-#pragma unroll
-    for (int i = 0; i < RC; ++i) {
-      const int row = r0 + i;
-      if (row >= r1) break;
-      const int s = sv.seq[row];
-      if (s != last) {
-        const int slot = sv.slots[s], row0 = sv.cu[s];
-        const int pos = sv.lens[slot] + row - row0;
-#pragma unroll
-        for (int j = 1; j < 4; ++j)
-          in[4 - j] = conv_in<T>(A, row, row0, pos, slot, j, c);
-        last = s;
-      }
-      in[0] = in[1];
-      in[1] = in[2];
-      in[2] = in[3];
-      in[3] = nx[i];
-      // in[0..2] are the three inputs before this one
-      float v = b;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) v = fmaf(w[j], in[j], v);
-      stf(u + (u64)row * A.C + c, v);
-    }
-    return;
-  }
-  for (int row = r0; row < r1; ++row) {
+  const int r1 = min((int)(blockIdx.y + 1) * RC, sv.n);
+  for (int row = blockIdx.y * RC; row < r1; ++row) {
     const int s = sv.seq[row], slot = sv.slots[s], row0 = sv.cu[s];
     stf(u + (u64)row * A.C + c,
         conv_at<T>(A, row, row0, sv.lens[slot] + row - row0, slot, c));
@@ -155,16 +204,27 @@ __global__ __launch_bounds__(256) void lru_gates_mfma(
       *(u32x4*)(us + r * ROW + e * 2) = d;
     }
     __syncthreads();
-#pragma unroll 2
-    for (int k = 0; k < kp; k += 32) {
-      const int kk = k + l4 * 8;
-      const s16x8 br = kk < kn ? *(const s16x8*)(wr + k0 + kk) : z8;
-      const s16x8 bi = kk < kn ? *(const s16x8*)(wi + k0 + kk) : z8;
+    constexpr int U = 4;         // steps loaded ahead of their products
+    for (int k = 0; k < kp; k += U * 32) {
+      s16x8 br[U], bi[U];
 #pragma unroll
-      for (int mt = 0; mt < 4; ++mt) {
-        const s16x8 a = *(const s16x8*)(us + (mt * 16 + l15) * ROW + kk * 2);
-        ar[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br, ar[mt], 0, 0, 0);
-        ai[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi, ai[mt], 0, 0, 0);
+      for (int i = 0; i < U; ++i) {
+        const int kk = k + i * 32 + l4 * 8;
+        br[i] = kk < kn ? *(const s16x8*)(wr + k0 + kk) : z8;
+        bi[i] = kk < kn ? *(const s16x8*)(wi + k0 + kk) : z8;
+      }
+#pragma unroll
+      for (int i = 0; i < U; ++i) {
+        if (k + i * 32 >= kp) break;
+        const int kk = k + i * 32 + l4 * 8;
+#pragma unroll
+        for (int mt = 0; mt < 4; ++mt) {
+          const s16x8 a = *(const s16x8*)(us + (mt * 16 + l15) * ROW + kk * 2);
+          ar[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br[i], ar[mt],
+                                                           0, 0, 0);
+          ai[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi[i], ai[mt],
+                                                           0, 0, 0);
+        }
       }
     }
   }
@@ -182,8 +242,8 @@ __global__ __launch_bounds__(256) void lru_gates_mfma(
       a[r] = 1.f;
       z[r] = 0.f;
       if (row < cnt)
-        lru_pair(ar[mt][r] + rb, ai[mt][r] + ib,
-                 ldf(u + (u64)(row0 + row) * A.C + c), csp, a[r], z[r]);
+        lru_pair<true>(ar[mt][r] + rb, ai[mt][r] + ib,
+                       ldf(u + (u64)(row0 + row) * A.C + c), csp, a[r], z[r]);
       if (r) {
         z[r] = fmaf(a[r], z[r - 1], z[r]);
         a[r] *= a[r - 1];
@@ -276,76 +336,123 @@ __global__ __launch_bounds__(256) void lru_apply_kernel(
     }
 #pragma unroll
     for (int i = 0; i < VEC; ++i)
-      y[i] = A.gain * fmaf(q[i].x, st[i], q[i].y) * gelu_tanh_f(y[i] + yb[i]);
+      y[i] = A.gain * fmaf(q[i].x, st[i], q[i].y) *
+             gelu_tanh_f<true>(y[i] + yb[i]);
     stv<bf16_t, VEC>((bf16_t*)A.out + (u64)row * A.ldo + c, y);
   }
 }
 
-// One token of up to 16 sequences x 16 channels of a block; the waves split
-// the gates' inner dimension.
+// One token of up to 16 sequences x CT * 16 channels of a block.  A wave has
+// 16 channels; with CT < 4 the waves also split the gates' inner dimension.
+constexpr int MAX_TAPS = 16;
+
+template <int CT>
 __global__ __launch_bounds__(256) void lru_step_mfma(SeqView sv, LruArgs A) {
-  constexpr int ROW = SKC * 2 + 16;
+  constexpr int ROW = SKC * 2 + 16, KW = 4 / CT, NC = CT * 16;
   __shared__ __attribute__((aligned(16))) char us[16 * ROW];
-  __shared__ float red[4][2][16][17];
+  __shared__ float red[KW][2][16][NC + 1];
+  __shared__ int back[MAX_TAPS][16];     // ring row of an earlier input, or -1
   const int b0 = blockIdx.z * 16, nb = min(16, sv.b - b0);
-  const int blk = blockIdx.y, n0 = blockIdx.x * 16;
+  const int blk = blockIdx.y, n0 = blockIdx.x * NC;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int l15 = lane & 15, l4 = lane >> 4;
-  const int ch = min(n0 + l15, A.n - 1);
+  const int ct = wave % CT, kw = wave / CT;
+  const int ch = min(n0 + ct * 16 + l15, A.n - 1);
   const bf16_t* wr = (const bf16_t*)A.gw + ((u64)blk * 2 * A.n + ch) * A.n;
   const bf16_t* wi = wr + (u64)A.n * A.n;
   const s16x8 z8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  for (int id = tid; id < 16 * A.taps; id += 256) {
+    const int i = id & 15, j = id >> 4;
+    if (i < nb) {
+      const int slot = sv.slots[b0 + i], p = sv.lens[slot] - j;
+      back[j][i] = p >= 0 ? slot * A.taps + p % A.taps : -1;
+    }
+  }
   f32x4 ar = {}, ai = {};
   for (int k0 = 0; k0 < A.n; k0 += SKC) {
     const int kn = min(SKC, A.n - k0), kp = (kn + 31) / 32 * 32;
     __syncthreads();
-    for (int id = tid; id < 16 * kp; id += 256) {
-      const int i = id / kp, k = id % kp;
-      unsigned short v = 0;
-      if (i < nb && k < kn) {
-        const int row = b0 + i, slot = sv.slots[row];
-        v = (unsigned short)f32_to_bf16_bits_rne(conv_at<bf16_t>(
-            A, row, row, sv.lens[slot], slot, blk * A.n + k0 + k));
+    for (int id = tid; id < nb * (kp / 4); id += 256) {
+      const int i = id / (kp / 4), k = (id % (kp / 4)) * 4;
+      float v[4] = {};
+      if (k < kn) {
+        const int c = blk * A.n + k0 + k;
+        float t[4], w[4];
+        ldf4(A.cb + c, v);
+        for (int j = A.taps - 1; j > 0; --j) {
+          const int row = back[j][i];
+          if (row < 0) continue;
+          ldf4(A.ring + (u64)row * A.C + c, t);
+          ldf4(A.cw + (u64)(A.taps - 1 - j) * A.C + c, w);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = fmaf(w[e], t[e], v[e]);
+        }
+        float xb[4];
+        load_x4<bf16_t>(A, b0 + i, c, t);
+        ldf4(A.xb + c, xb);
+        ldf4(A.cw + (u64)(A.taps - 1) * A.C + c, w);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = fmaf(w[e], t[e] + xb[e], v[e]);
       }
-      *(unsigned short*)(us + i * ROW + k * 2) = v;
+      stf4((bf16_t*)(us + i * ROW) + k, v);
     }
     __syncthreads();
-#pragma unroll 2
-    for (int k = wave * 32; k < kp; k += 128) {
-      const int kk = k + l4 * 8;
-      const s16x8 br = kk < kn ? *(const s16x8*)(wr + k0 + kk) : z8;
-      const s16x8 bi = kk < kn ? *(const s16x8*)(wi + k0 + kk) : z8;
-      const s16x8 a = *(const s16x8*)(us + l15 * ROW + kk * 2);
-      ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br, ar, 0, 0, 0);
-      ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi, ai, 0, 0, 0);
+    constexpr int U = CT == 4 ? 8 : 2;
+    for (int k = kw * 32; k < kp; k += U * KW * 32) {
+      s16x8 br[U], bi[U];
+#pragma unroll
+      for (int i = 0; i < U; ++i) {
+        const int kk = k + i * KW * 32 + l4 * 8;
+        br[i] = kk < kn ? *(const s16x8*)(wr + k0 + kk) : z8;
+        bi[i] = kk < kn ? *(const s16x8*)(wi + k0 + kk) : z8;
+      }
+#pragma unroll
+      for (int i = 0; i < U; ++i) {
+        const int kk = k + i * KW * 32 + l4 * 8;
+        const s16x8 a = l15 < nb && kk < kp
+                            ? *(const s16x8*)(us + l15 * ROW + kk * 2)
+                            : z8;
+        ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, br[i], ar, 0, 0, 0);
+        ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, bi[i], ai, 0, 0, 0);
+      }
     }
   }
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    red[wave][0][l4 * 4 + r][l15] = ar[r];
-    red[wave][1][l4 * 4 + r][l15] = ai[r];
+    red[kw][0][l4 * 4 + r][ct * 16 + l15] = ar[r];
+    red[kw][1][l4 * 4 + r][ct * 16 + l15] = ai[r];
   }
   __syncthreads();
-  const int i = tid >> 4, j = n0 + (tid & 15);
-  if (i >= nb || j >= A.n) return;
-  float r = A.gb[(u64)blk * 2 * A.n + j], g = A.gb[((u64)blk * 2 + 1) * A.n + j];
+  for (int id = tid; id < nb * NC; id += 256) {
+    const int i = id / NC, j = id % NC;
+    if (n0 + j >= A.n) continue;
+    float r = A.gb[(u64)blk * 2 * A.n + n0 + j];
+    float g = A.gb[((u64)blk * 2 + 1) * A.n + n0 + j];
 #pragma unroll
-  for (int w = 0; w < 4; ++w) {
-    r += red[w][0][i][tid & 15];
-    g += red[w][1][i][tid & 15];
+    for (int w = 0; w < KW; ++w) {
+      r += red[w][0][i][j];
+      g += red[w][1][i][j];
+    }
+    const int row = b0 + i, slot = sv.slots[row], pos = sv.lens[slot];
+    const int c = blk * A.n + n0 + j;
+    const float x = ldf((const bf16_t*)A.x + (u64)row * A.ld + c) + A.xb[c];
+    float u = A.cb[c];
+    for (int t = A.taps - 1; t > 0; --t)
+      if (back[t][i] >= 0)
+        u = fmaf(A.cw[(u64)(A.taps - 1 - t) * A.C + c],
+                 A.ring[(u64)back[t][i] * A.C + c], u);
+    u = fmaf(A.cw[(u64)(A.taps - 1) * A.C + c], x, u);
+    float a, z;
+    lru_pair<true>(r, g, round_to(u, (const bf16_t*)nullptr),
+                   A.c * softplus_f(A.lam[c]), a, z);
+    float* sp = A.S + (u64)slot * A.C + c;
+    const float S = fmaf(a, pos == 0 ? 0.f : *sp, z);
+    *sp = S;
+    A.ring[(u64)back[0][i] * A.C + c] = x;     // no one reads this row
+    const float y = ldf((const bf16_t*)A.y + (u64)row * A.ld + c) + A.yb[c];
+    stf((bf16_t*)A.out + (u64)row * A.ldo + c,
+        A.gain * S * gelu_tanh_f<true>(y));
   }
-  const int row = b0 + i, slot = sv.slots[row], pos = sv.lens[slot];
-  const int c = blk * A.n + j;
-  float a, z;
-  lru_pair(r, g, conv_at<bf16_t>(A, row, row, pos, slot, c),
-           A.c * softplus_f(A.lam[c]), a, z);
-  float* sp = A.S + (u64)slot * A.C + c;
-  const float S = fmaf(a, pos == 0 ? 0.f : *sp, z);
-  *sp = S;
-  A.ring[((u64)slot * A.taps + pos % A.taps) * A.C + c] =
-      ldf((const bf16_t*)A.x + (u64)row * A.ld + c) + A.xb[c];
-  const float y = ldf((const bf16_t*)A.y + (u64)row * A.ld + c) + A.yb[c];
-  stf((bf16_t*)A.out + (u64)row * A.ldo + c, A.gain * S * gelu_tanh_f(y));
 }
 
 // any size: a workgroup = one row of one block, a wave a channel at a time
@@ -371,7 +478,7 @@ __global__ __launch_bounds__(256) void lru_gates_any(
     if (lane == 0) {
       const int c = blk * A.n + j;
       float a, z;
-      lru_pair(r, g, ub[j], A.c * softplus_f(A.lam[c]), a, z);
+      lru_pair<false>(r, g, ub[j], A.c * softplus_f(A.lam[c]), a, z);
       ab[(u64)row * A.C + c] = make_float2(a, z);
     }
   }
@@ -390,7 +497,7 @@ __global__ __launch_bounds__(64) void lru_scan_kernel(
     const float2 p = ab[(u64)row * A.C + c];
     S = fmaf(p.x, S, p.y);
     const float y = ldf((const T*)A.y + (u64)row * A.ld + c) + A.yb[c];
-    stf((T*)A.out + (u64)row * A.ldo + c, A.gain * S * gelu_tanh_f(y));
+    stf((T*)A.out + (u64)row * A.ldo + c, A.gain * S * gelu_tanh_f<false>(y));
   }
   A.S[(u64)slot * A.C + c] = S;
   keep_inputs<T>(sv, A, s, slot, c);
@@ -403,13 +510,14 @@ LruArgs args(const void* x, const void* y, long ld, const void* xb,
   return LruArgs{x, y, (u64)ld, (const float*)xb, (const float*)yb,
                  (const float*)cw, (const float*)cb, (const float*)gb,
                  (const float*)lam, gw, (float*)ring, (float*)S, out,
-                 (u64)ldo, C, blocks, C / blocks, taps, c, gain};
+                 (u64)ldo, C, blocks, C / blocks, taps, c, gain,
+                 ld % 4 == 0 && ((u64)x & 15) == 0};
 }
 
 }  // namespace
 
-bool lfmq_lru_mfma_ok(const void* gw, int n) {
-  return n % 8 == 0 && ((u64)gw & 15) == 0;
+bool lfmq_lru_mfma_ok(const void* gw, int n, int taps) {
+  return n % 8 == 0 && taps <= MAX_TAPS && ((u64)gw & 15) == 0;
 }
 
 // prompts: u [n, C], ab [n, C, 2], ends [tiles, C, 2] scratch; tile0 [b]
@@ -427,19 +535,33 @@ hipError_t lfmq_gated_lru(const SeqView& sv, const void* x, const void* y,
   const LruArgs A = args(x, y, ld, xb, yb, cw, cb, gw, gb, lam, ring, S, out,
                          ldo, C, blocks, taps, c, gain);
   if (mfma && single) {
-    hipLaunchKernelGGL(lru_step_mfma,
-                       dim3((A.n + 15) / 16, blocks, (sv.b + 15) / 16),
-                       dim3(256), 0, stream, sv, A);
+    // wide tiles compute each convolution output less often, narrow ones
+    // spread few sequences over the chip
+    if (sv.b >= 16)
+      hipLaunchKernelGGL(lru_step_mfma<4>,
+                         dim3((A.n + 63) / 64, blocks, (sv.b + 15) / 16),
+                         dim3(256), 0, stream, sv, A);
+    else
+      hipLaunchKernelGGL(lru_step_mfma<1>,
+                         dim3((A.n + 15) / 16, blocks, 1), dim3(256), 0,
+                         stream, sv, A);
     return hipGetLastError();
   }
-  const dim3 conv_grid((C + 255) / 256, (sv.n + RC - 1) / RC);
+  const bool c4 = taps == 4 && C % 4 == 0;
+  const int per = c4 ? 1024 : 256;
+  const dim3 conv_grid((C + per - 1) / per, (sv.n + RC - 1) / RC);
   if (conv_grid.y > 65535) return hipErrorInvalidValue;
-  if (f32)
-    hipLaunchKernelGGL(lru_conv_kernel<float>, conv_grid, dim3(256), 0,
-                       stream, sv, A, (float*)u);
-  else
-    hipLaunchKernelGGL(lru_conv_kernel<bf16_t>, conv_grid, dim3(256), 0,
-                       stream, sv, A, (bf16_t*)u);
+#define CONV(T)                                                              \
+  do {                                                                       \
+    if (c4)                                                                  \
+      hipLaunchKernelGGL(lru_conv4_kernel<T>, conv_grid, dim3(256), 0,       \
+                         stream, sv, A, (T*)u);                              \
+    else                                                                     \
+      hipLaunchKernelGGL(lru_conv_kernel<T>, conv_grid, dim3(256), 0,        \
+                         stream, sv, A, (T*)u);                              \
+  } while (0)
+  if (f32) CONV(float); else CONV(bf16_t);
+#undef CONV
   const dim3 chan_grid((C + 63) / 64, sv.b);
   if (mfma) {
     hipLaunchKernelGGL(lru_gates_mfma,
@@ -451,8 +573,8 @@ hipError_t lfmq_gated_lru(const SeqView& sv, const void* x, const void* y,
                        A, (const i32*)tile0, (float2*)ends);
     const bool v4 = C % 4 == 0 && ld % 4 == 0 && ldo % 4 == 0 &&
                     (((u64)y | (u64)out) & 7) == 0 && ((u64)yb & 15) == 0;
-    const int per = v4 ? 1024 : 256;
-    const dim3 ag((C + per - 1) / per, (sv.n + RC - 1) / RC);
+    const int ap = v4 ? 1024 : 256;
+    const dim3 ag((C + ap - 1) / ap, (sv.n + RC - 1) / RC);
     if (v4)
       hipLaunchKernelGGL(lru_apply_kernel<4>, ag, dim3(256), 0, stream, sv, A,
                          (const i32*)tile0, (const float2*)ab,

@@ -23,7 +23,8 @@ namespace {
 // routing
 // ---------------------------------------------------------------------------
 
-constexpr int RT = 512, RW = RT / 64, RROWS = 16;
+constexpr int RT = 1024, RW = RT / 64, RROWS = 16;
+constexpr int EG = 32;      // experts a pass over the router's matrix
 
 struct RouteArgs {
   const void *h, *w;      // w [E + has_sg, width]
@@ -91,7 +92,7 @@ __global__ __launch_bounds__(RT) void moe_route_kernel(RouteArgs A) {
   extern __shared__ float sh[];
   const int E1 = A.E + (A.sg != nullptr);
   float* lg = sh;                      // [RROWS][E1]
-  float* red = sh + RROWS * E1;        // MF: [RW][16][64]
+  float* red = sh + RROWS * E1;        // MF: [RW][16][EG]
   const int r0 = blockIdx.x * RROWS;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const T* h = (const T*)A.h;
@@ -100,38 +101,45 @@ __global__ __launch_bounds__(RT) void moe_route_kernel(RouteArgs A) {
     const int l15 = lane & 15, l4 = lane >> 4;
     const T* hr = h + (u64)min(r0 + l15, A.n - 1) * A.width;
     const s16x8 z8 = {0, 0, 0, 0, 0, 0, 0, 0};
-    for (int e0 = 0; e0 < E1; e0 += 64) {
-      f32x4 acc[4] = {};
-      const T* wr[4];
+    for (int e0 = 0; e0 < E1; e0 += EG) {
+      f32x4 acc[EG / 16] = {};
+      const T* wr[EG / 16];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < EG / 16; ++j)
         wr[j] = w + (u64)min(e0 + j * 16 + l15, E1 - 1) * A.width;
-#pragma unroll 2
-      for (int k = wave * 32; k < A.width; k += RW * 32) {
-        const int kk = k + l4 * 8;
-        const bool ok = kk < A.width;
-        const s16x8 a = ok ? *(const s16x8*)(hr + kk) : z8;
+      constexpr int U = 4;       // steps loaded ahead of their products
+      for (int k = wave * 32; k < A.width; k += U * RW * 32) {
+        s16x8 a[U], b[U][EG / 16];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          if (e0 + j * 16 >= E1) break;
-          const s16x8 b = ok ? *(const s16x8*)(wr[j] + kk) : z8;
-          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[j], 0, 0, 0);
+        for (int i = 0; i < U; ++i) {
+          const int kk = k + i * RW * 32 + l4 * 8;
+          const bool ok = kk < A.width;
+          a[i] = ok ? *(const s16x8*)(hr + kk) : z8;
+#pragma unroll
+          for (int j = 0; j < EG / 16; ++j)
+            b[i][j] = ok ? *(const s16x8*)(wr[j] + kk) : z8;
         }
+#pragma unroll
+        for (int i = 0; i < U; ++i)
+#pragma unroll
+          for (int j = 0; j < EG / 16; ++j)
+            acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[i][j],
+                                                             acc[j], 0, 0, 0);
       }
       __syncthreads();
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < EG / 16; ++j)
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          red[(wave * 16 + l4 * 4 + r) * 64 + j * 16 + l15] = acc[j][r];
+          red[(wave * 16 + l4 * 4 + r) * EG + j * 16 + l15] = acc[j][r];
       __syncthreads();
-      for (int id = tid; id < 16 * 64; id += RT) {
-        const int e = e0 + (id & 63);
+      for (int id = tid; id < 16 * EG; id += RT) {
+        const int e = e0 + id % EG;
         if (e >= E1) continue;
         float v = 0.f;
 #pragma unroll
-        for (int g = 0; g < RW; ++g) v += red[g * 1024 + id];
-        lg[(id >> 6) * E1 + e] = v;
+        for (int g = 0; g < RW; ++g) v += red[g * 16 * EG + id];
+        lg[id / EG * E1 + e] = v;
       }
     }
   } else {
@@ -200,10 +208,15 @@ struct GemmArgs {
   float limit, alpha, beta;
 };
 
+// T: the storage type (16-bit results take the hardware's exponential)
+template <typename T>
 __device__ __forceinline__ float glu_f(float g, float u, const GemmArgs& A) {
   g = fminf(g, A.limit);
   u = fminf(fmaxf(u, -A.limit), A.limit);
-  return g * sigmoid_f(A.alpha * g) * (u + A.beta);
+  const float s = sizeof(T) == 2
+                      ? __builtin_amdgcn_rcpf(1.f + __expf(-A.alpha * g))
+                      : sigmoid_f(A.alpha * g);
+  return g * s * (u + A.beta);
 }
 
 // 16 rows x 16 columns; NW waves split K in pairs of 32
@@ -227,19 +240,24 @@ __global__ __launch_bounds__(NW * 64) void moe_rows16(GemmArgs A) {
   if constexpr (GLU) wr[1] = w + (u64)(A.N + n) * A.K;
   const s16x8 z8 = {0, 0, 0, 0, 0, 0, 0, 0};
   f32x4 acc[NB] = {};
-#pragma unroll 4
-  for (int k = wave * 64; k < A.K; k += NW * 64) {
+  constexpr int U = 8;           // steps loaded ahead of their products
+  for (int k = wave * 64; k < A.K; k += U / 2 * NW * 64) {
+    s16x8 a[U], b[U][NB];
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int kk = k + i * 32 + l4 * 8;
+    for (int i = 0; i < U; ++i) {
+      const int kk = k + (i >> 1) * NW * 64 + (i & 1) * 32 + l4 * 8;
       const bool ok = kk < A.K;
-      const s16x8 a = ok ? *(const s16x8*)(ar + kk) : z8;
+      a[i] = ok ? *(const s16x8*)(ar + kk) : z8;
 #pragma unroll
-      for (int j = 0; j < NB; ++j) {
-        const s16x8 b = ok ? *(const s16x8*)(wr[j] + kk) : z8;
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[j], 0, 0, 0);
-      }
+      for (int j = 0; j < NB; ++j)
+        b[i][j] = ok ? *(const s16x8*)(wr[j] + kk) : z8;
     }
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+#pragma unroll
+      for (int j = 0; j < NB; ++j)
+        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[i][j], acc[j],
+                                                         0, 0, 0);
   }
 #pragma unroll
   for (int j = 0; j < NB; ++j)
@@ -258,7 +276,7 @@ __global__ __launch_bounds__(NW * 64) void moe_rows16(GemmArgs A) {
   float o = v[0];
   if constexpr (GLU) {
     const float s = A.weight != nullptr ? A.weight[row0 + i] : 1.f;
-    o = glu_f(s * v[0], s * v[1], A);
+    o = glu_f<bf16_t>(s * v[0], s * v[1], A);
   }
   stf((bf16_t*)A.out + (u64)(row0 + i) * A.N + n0 + c, o);
 }
@@ -359,7 +377,8 @@ __global__ __launch_bounds__(256, 2) void moe_rows128(GemmArgs A) {
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
           const int n = n0 + wn * 32 + j * 16 + l15;
-          if (n < A.N) stf(o + n, glu_f(s * acc[i][j][r], s * acc[i][j + 2][r], A));
+          if (n < A.N) stf(o + n, glu_f<bf16_t>(s * acc[i][j][r],
+                                               s * acc[i][j + 2][r], A));
         }
       } else {
 #pragma unroll
@@ -395,7 +414,7 @@ __global__ __launch_bounds__(256) void moe_any(GemmArgs A) {
       if (GLU) {
         u = wave_reduce_sum(u);
         const float s = A.weight != nullptr ? A.weight[slot] : 1.f;
-        v = glu_f(s * v, s * u, A);
+        v = glu_f<T>(s * v, s * u, A);
       }
       if (lane == 0) stf((T*)A.out + (u64)slot * A.N + n, v);
     }
@@ -403,17 +422,23 @@ __global__ __launch_bounds__(256) void moe_any(GemmArgs A) {
 }
 
 // the same activation on a fused [gate | up] row
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void clamped_glu_kernel(
     const T* __restrict__ gu, T* __restrict__ y, u64 rows, int ff,
     GemmArgs A) {
-  const u64 total = rows * ff;
+  const u64 total = rows * ff / VEC;
+  const int per = ff / VEC;
   for (u64 id = (u64)blockIdx.x * 256 + threadIdx.x; id < total;
        id += (u64)gridDim.x * 256) {
-    const u64 row = id / ff;
-    const int j = id % ff;
+    const u64 row = id / per;
+    const int j = id % per * VEC;
     const T* p = gu + row * 2 * ff + j;
-    stf(y + id, glu_f(ldf(p), ldf(p + ff), A));
+    float g[VEC], u[VEC];
+    ldv<T, VEC>(p, g);
+    ldv<T, VEC>(p + ff, u);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) g[e] = glu_f<T>(g[e], u[e], A);
+    stv<T, VEC>(y + row * ff + j, g);
   }
 }
 
@@ -455,7 +480,7 @@ hipError_t lfmq_moe_route_sort(const void* h, const void* w, void* ids,
               (i32*)pos, (float*)weight, (i32*)tiles, n, width, E, top, bm,
               max_tiles};
   const int E1 = E + (sg != nullptr);
-  const size_t lds = sizeof(float) * (size_t)(RROWS * E1 + (mfma ? RW * 1024 : 0));
+  const size_t lds = sizeof(float) * (size_t)(RROWS * E1 + (mfma ? RW * 16 * EG : 0));
   if (lds > 64 * 1024 || top > E) return hipErrorInvalidValue;
   const dim3 grid((n + RROWS - 1) / RROWS), block(RT);
   if (f32)
@@ -494,14 +519,14 @@ hipError_t lfmq_clamped_glu(const void* gu, void* y, long rows, int ff,
   A.limit = limit;
   A.alpha = alpha;
   A.beta = beta;
-  const u64 want = ((u64)rows * ff + 255) / 256;
-  const u32 grid = (u32)(want < 4096 ? want : 4096);
-  if (f32)
-    hipLaunchKernelGGL(clamped_glu_kernel<float>, dim3(grid), dim3(256), 0,
-                       stream, (const float*)gu, (float*)y, (u64)rows, ff, A);
-  else
-    hipLaunchKernelGGL(clamped_glu_kernel<bf16_t>, dim3(grid), dim3(256), 0,
-                       stream, (const bf16_t*)gu, (bf16_t*)y, (u64)rows, ff,
-                       A);
+  const bool v4 = ff % 4 == 0 && (((u64)gu | (u64)y) & 15) == 0;
+  const u64 want = ((u64)rows * ff / (v4 ? 4 : 1) + 255) / 256;
+  const dim3 grid((u32)(want < 8192 ? want : 8192));
+#define GO(T, V)                                                             \
+  hipLaunchKernelGGL((clamped_glu_kernel<T, V>), grid, dim3(256), 0, stream, \
+                     (const T*)gu, (T*)y, (u64)rows, ff, A)
+  if (f32) { if (v4) GO(float, 4); else GO(float, 1); }
+  else { if (v4) GO(bf16_t, 4); else GO(bf16_t, 1); }
+#undef GO
   return hipGetLastError();
 }

@@ -66,6 +66,13 @@ __global__ __launch_bounds__(512) void post_norm_kernel(PostArgs A) {
       const int64_t t = A.tok[row];
       src += (u64)(t < 0 ? 0 : (t >= A.vocab ? A.vocab - 1 : t)) * width;
     }
+    constexpr int PK = 8;           // choices kept in registers
+    u64 at[PK] = {};
+    if constexpr (SRC == EXPERTS) {
+#pragma unroll
+      for (int k = 0; k < PK; ++k)
+        if (k < A.top) at[k] = (u64)A.pos[(u64)row * A.top + k] * width;
+    }
     const float sg =
         SRC == EXPERTS && A.shared != nullptr ? A.sgate[row] : 0.f;
     for (int j = t0; j < width; j += step) {
@@ -73,7 +80,15 @@ __global__ __launch_bounds__(512) void post_norm_kernel(PostArgs A) {
       if constexpr (SRC == EXPERTS) {
 #pragma unroll
         for (int e = 0; e < VEC; ++e) a[e] = 0.f;
-        for (int k = 0; k < A.top; ++k) {
+#pragma unroll
+        for (int k = 0; k < PK; ++k) {
+          if (k >= A.top) break;
+          float c[VEC];
+          ldv<T, VEC>(src + at[k] + j, c);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) a[e] += c[e];
+        }
+        for (int k = PK; k < A.top; ++k) {
           float c[VEC];
           ldv<T, VEC>(src + (u64)A.pos[(u64)row * A.top + k] * width + j, c);
 #pragma unroll

@@ -11,9 +11,7 @@
 
 namespace {
 
-constexpr int TPB = 256;
-
-template <typename T, int VEC>
+template <typename T, int VEC, int TPB>
 __global__ __launch_bounds__(TPB) void qk_prep_kernel(
     const T* __restrict__ in, u64 ld, SeqView sv,
     const float* __restrict__ wq, const float* __restrict__ wk,
@@ -104,13 +102,17 @@ hipError_t lfmq_qk_prep(const void* in, long ld, const SeqView& sv,
   const bool v4 = ((ld | dim | half | nv) & 3) == 0 &&
                   (((u64)in | (u64)wq | (u64)wk | (u64)q | (u64)kc |
                     (u64)vc) & 15) == 0;
+  // few rows: more threads each
 #define GO(T, V)                                                             \
-  hipLaunchKernelGGL((qk_prep_kernel<T, V>), dim3(sv.n), dim3(TPB), lds,     \
+  do { if (sv.n < 512) GOT(T, V, 1024); else GOT(T, V, 256); } while (0)
+#define GOT(T, V, N)                                                         \
+  hipLaunchKernelGGL((qk_prep_kernel<T, V, N>), dim3(sv.n), dim3(N), lds,    \
                      stream, (const T*)in, (u64)ld, sv, (const float*)wq,    \
                      (const float*)wk, (const float*)inv_freq, (T*)q,        \
                      (T*)kc, (T*)vc, cap, nq, nk, nv, dim, half, eps)
   if (f32) { if (v4) GO(float, 4); else GO(float, 1); }
   else { if (v4) GO(bf16_t, 4); else GO(bf16_t, 1); }
+#undef GOT
 #undef GO
   return hipGetLastError();
 }

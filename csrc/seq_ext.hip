@@ -88,7 +88,7 @@ hipError_t lfmq_attn_grouped_decode(const void*, const void*, const void*,
                                     const SeqView&, const void*, void*, void*,
                                     long, int, int, int, int, int, int, float,
                                     float, hipStream_t);
-bool lfmq_lru_mfma_ok(const void*, int);
+bool lfmq_lru_mfma_ok(const void*, int, int);
 hipError_t lfmq_gated_lru(const SeqView&, const void*, const void*, long,
                           const void*, const void*, const void*, const void*,
                           const void*, const void*, const void*, void*, void*,
@@ -659,7 +659,7 @@ void attn_grouped(T_ q, T_ kc, T_ vc, T_ seq, T_ cu, T_ slots, T_ lens,
 }
 
 // x and y: column views of one projection [N, *]; gw [blocks, 2, n, n],
-// gb [blocks, 2, n]; ring [slots, taps, C], S [slots, C].  tile0 [b] first
+// gb [blocks, 2, n]; cw [taps, C], ring [slots, taps, C], S [slots, C].  tile0 [b] first
 // 64-token tile of each sequence, `tiles` in all.
 void gated_lru(T_ x, T_ y, T_ seq, T_ cu, T_ slots, T_ lens, T_ xb, T_ yb,
                T_ cw, T_ cb, T_ gw, T_ gb, T_ lam, T_ ring, T_ S, T_ out,
@@ -684,7 +684,8 @@ void gated_lru(T_ x, T_ y, T_ seq, T_ cu, T_ slots, T_ lens, T_ xb, T_ yb,
               "gated_lru: shape mismatch");
   const long taps = ring.size(1);
   const bool mfma =
-      !f32 && !general && lfmq_lru_mfma_ok(gw.data_ptr(), (int)n);
+      !f32 && !general && lfmq_lru_mfma_ok(gw.data_ptr(), (int)n, (int)taps) &&
+      al16(cw) && al16(cb) && al16(xb) && al16(ring);
   const bool single = sv.n == sv.b && max_count == 1;
   T_ u, ab, ends;
   if (!(mfma && single)) {

@@ -1,7 +1,7 @@
-"""Throughput of one architecture beside another at equal layer sizes.
+"""Throughput of architectures side by side at equal layer sizes.
 
-bf16 weights on both sides, random; prefill (whole prompt, all logits) and
-graph-captured greedy decode at a given context length.  Both models are
+bf16 weights everywhere, random; prefill (whole prompt, all logits) and
+graph-captured greedy decode at a given context length.  All models are
 resident and timed in turn, `repeats` times each; the best time counts.
 """
 from __future__ import annotations
@@ -14,23 +14,27 @@ from ..api import build_model
 from ..models.graph import GraphDecoder
 from ..models.llama import LlamaConfig
 from ..models.rapivik import RapivikConfig
+from ..models.zatasun import ZatasunConfig
 from .decode import _fast_random_init
 
-# width-alike pairs; depth and vocab cut so that a run takes seconds
+# alike in width and in the parameters a token meets; depth and vocab cut so that a run takes seconds
 SIZES = {
     "2k": dict(
         llama=lambda n: LlamaConfig(
             vocab_size=32000, hidden_size=2048, intermediate_size=8192,
             n_layers=n, n_heads=16, n_kv_heads=4, head_dim=128),
-        rapivik=lambda n: RapivikConfig.sized_1b(n_layers=n)),
+        rapivik=lambda n: RapivikConfig.sized_1b(n_layers=n),
+        zatasun=lambda n: ZatasunConfig.sized_1b(n_layers=n)),
     "4k": dict(
         llama=lambda n: LlamaConfig(
             vocab_size=32000, hidden_size=4096, intermediate_size=14336,
             n_layers=n, n_heads=32, n_kv_heads=8, head_dim=128),
-        rapivik=lambda n: RapivikConfig.sized_8b(n_layers=n, vocab=32000)),
+        rapivik=lambda n: RapivikConfig.sized_8b(n_layers=n, vocab=32000),
+        zatasun=lambda n: ZatasunConfig.sized_8b(n_layers=n, vocab=32000)),
     "tiny-debug": dict(
         llama=lambda n: LlamaConfig.tiny(n_layers=n),
-        rapivik=lambda n: RapivikConfig.tiny(n_layers=n)),
+        rapivik=lambda n: RapivikConfig.tiny(n_layers=n),
+        zatasun=lambda n: ZatasunConfig.tiny(n_layers=n)),
 }
 PREFILL = ((1, 2048), (1, 8192), (8, 1024))      # batch, prompt
 DECODE = ((1, 1024), (1, 8192), (16, 1024), (64, 2048))
@@ -74,22 +78,37 @@ def decode_tok_s(model, batch: int, context: int, steps: int,
     return batch * steps / best
 
 
-def compare(size: str, n_layers: int, steps: int = 64, repeats: int = 3,
-            prefill=PREFILL, decode=DECODE):
-    """Yields one dict per (phase, shape) with both models' tokens/s."""
-    models = {k: _build(f(n_layers), "cuda") for k, f in SIZES[size].items()}
-    params = {k: sum(p.numel() for n, p in m.named_parameters()
-                     if not n.startswith(("embed", "bigram", "lm_head"))) / 1e6
-              for k, m in models.items()}          # of the layers
+def layer_params(model) -> tuple:
+    """(all, met by one token) parameters of the layers."""
+    total = active = 0
+    for name, p in model.named_parameters():
+        if name.startswith(("embed", "bigram", "lm_head")):
+            continue
+        total += p.numel()
+        part = 1.0
+        if name.endswith((".gate_up", ".down")):     # stacked experts
+            moe = model.get_submodule(name.rpartition(".")[0])
+            part = moe.top / moe.experts
+        active += p.numel() * part
+    return total, active
+
+
+def compare(size: str, n_layers: int, models=("llama", "rapivik"),
+            steps: int = 64, repeats: int = 3, prefill=PREFILL,
+            decode=DECODE):
+    """Yields one dict per (phase, shape) with every model's tokens/s; ratio
+    is the last one's to the first one's."""
+    built = {k: _build(SIZES[size][k](n_layers), "cuda") for k in models}
+    params = {k: [round(v / 1e6) for v in layer_params(m)]
+              for k, m in built.items()}
     for phase, shapes in (("prefill", prefill), ("decode", decode)):
         for b, s in shapes:
             row = {"size": size, "layers": n_layers, "phase": phase,
-                   "batch": b, "length": s,
-                   "mparams": {k: round(v) for k, v in params.items()}}
-            for name, m in models.items():
+                   "batch": b, "length": s, "mparams_all_active": params}
+            for name, m in built.items():
                 row[name] = round(
                     prefill_tok_s(m, b, s, repeats) if phase == "prefill"
                     else decode_tok_s(m, b, s, steps, repeats), 1)
                 torch.cuda.empty_cache()
-            row["ratio"] = round(row["rapivik"] / row["llama"], 3)
+            row["ratio"] = round(row[models[-1]] / row[models[0]], 3)
             yield row

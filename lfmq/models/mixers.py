@@ -217,7 +217,8 @@ class GatedLRU(nn.Module):
         self.width, self.taps = width, taps
         self.rows_in, self.rows_out = 2 * width, width    # [gelu | conv]
         self.y_b, self.x_b = _fp32(width), _fp32(width)
-        self.conv_w = nn.Parameter(torch.zeros(width, taps))
+        # rows by age, the current token's last
+        self.conv_w = nn.Parameter(torch.zeros(taps, width))
         self.conv_b = _fp32(width)
         # [recurrence gate | input gate] of every block, [out, in]
         self.gate_w = nn.Parameter(torch.zeros(blocks, 2, n, n, dtype=dtype))

@@ -13,10 +13,13 @@ from typing import Callable, Optional
 
 import torch
 
-from . import rapivik, zatasun
 from .llama import LlamaConfig, LlamaForCausalLM
 from .mixtral import MixtralConfig, MixtralForCausalLM
 from .opt import OPTConfig, OPTForCausalLM
+from .rapivik import RapivikConfig, RapivikForCausalLM
+from .rapivik import convert_state as rapivik_state
+from .zatasun import ZatasunConfig, ZatasunForCausalLM
+from .zatasun import convert_state as zatasun_state
 
 
 @dataclass(frozen=True)
@@ -32,10 +35,10 @@ ARCHS = {
     "llama": ArchSpec(LlamaConfig, LlamaForCausalLM, torch.bfloat16),
     "opt": ArchSpec(OPTConfig, OPTForCausalLM, torch.float32),
     "mixtral": ArchSpec(MixtralConfig, MixtralForCausalLM, torch.bfloat16),
-    "rapivik": ArchSpec(rapivik.RapivikConfig, rapivik.RapivikForCausalLM,
-                        torch.bfloat16, rapivik.convert_state),
-    "zatasun": ArchSpec(zatasun.ZatasunConfig, zatasun.ZatasunForCausalLM,
-                        torch.bfloat16, zatasun.convert_state),
+    "rapivik": ArchSpec(RapivikConfig, RapivikForCausalLM, torch.bfloat16,
+                        rapivik_state),
+    "zatasun": ArchSpec(ZatasunConfig, ZatasunForCausalLM, torch.bfloat16,
+                        zatasun_state),
 }
 
 

@@ -193,7 +193,7 @@ def convert_state(cfg: ZatasunConfig, src: Dict[str, torch.Tensor]
 
     def recurrence(p, o):
         out[o + "y_b"], out[o + "x_b"] = src.pop(p + "y.b"), src.pop(p + "x.b")
-        out[o + "conv_w"] = src.pop(p + "conv")
+        out[o + "conv_w"] = src.pop(p + "conv").t().contiguous()
         out[o + "conv_b"] = src.pop(p + "conv.b")
         out[o + "gate_w"] = torch.stack([src.pop(p + "ra"),
                                          src.pop(p + "ri")], 1)

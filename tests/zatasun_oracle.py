@@ -52,15 +52,14 @@ def frequencies(dims, base, scaling=None):
 
 
 def rotate(x, pos, freqs):
-    """x [..., dim]: pairs (i, i + len(freqs)) turn by pos * freqs[i]."""
-    y = x.clone()
-    n = len(freqs)
-    for i, f in enumerate(freqs):
-        c, s = math.cos(pos * f), math.sin(pos * f)
-        u, v = x[..., i], x[..., i + n]
-        y[..., i] = u * c - v * s
-        y[..., i + n] = v * c + u * s
-    return y
+    """x [..., dim] at position(s) pos (a number, or one per leading index):
+    pairs (i, i + len(freqs)) turn by pos * freqs[i]."""
+    n, f = len(freqs), torch.tensor(freqs, dtype=x.dtype)
+    p = torch.as_tensor(pos, dtype=x.dtype)
+    a = p.reshape(p.shape + (1,) * (x.dim() - p.dim())) * f
+    u, v = x[..., :n], x[..., n:2 * n]
+    return torch.cat([u * torch.cos(a) - v * torch.sin(a),
+                      v * torch.cos(a) + u * torch.sin(a), x[..., 2 * n:]], -1)
 
 
 # ---- attention -----------------------------------------------------------------
@@ -72,7 +71,7 @@ def sink_attend(scores, values, sink):
     return (e @ values) / (e.sum() + torch.exp(sink - top))
 
 
-def attention(q, k, v, wq, wk, sink, m, eps, pos0=0):
+def attention(q, k, v, wq, wk, sink, m, eps):
     """Projections [T, ...] of one whole sequence -> [T, heads * vdim]."""
     H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     f = frequencies(m["rot"]["dims"], m["rot"]["base"],
@@ -81,8 +80,8 @@ def attention(q, k, v, wq, wk, sink, m, eps, pos0=0):
     q = (rms(q, eps) * wq).view(T, H, d)
     k = (rms(k, eps) * wk).view(T, G, d)
     v = v.view(T, G, dv)
-    q = torch.stack([rotate(q[t], pos0 + t, f) for t in range(T)])
-    k = torch.stack([rotate(k[t], pos0 + t, f) for t in range(T)])
+    pos = torch.arange(T)
+    q, k = rotate(q, pos, f), rotate(k, pos, f)
     out = torch.empty(T, H, dv, dtype=q.dtype)
     for h in range(H):
         g = h // (H // G)
