@@ -342,13 +342,16 @@ __global__ __launch_bounds__(256) void lru_apply_kernel(
   }
 }
 
-// One token of up to 16 sequences x CT * 16 channels of a block.  A wave has
-// 16 channels; with CT < 4 the waves also split the gates' inner dimension.
+// One token of up to 16 sequences x CT * 16 channels of a block: a wave has
+// 16 channels and a quarter of the gates' inner dimension.  TAPS 0: any
+// number of them.
 constexpr int MAX_TAPS = 16;
 
-template <int CT>
-__global__ __launch_bounds__(256) void lru_step_mfma(SeqView sv, LruArgs A) {
-  constexpr int ROW = SKC * 2 + 16, KW = 4 / CT, NC = CT * 16;
+template <int CT, int TAPS>
+__global__ __launch_bounds__(CT * 256) void lru_step_mfma(SeqView sv,
+                                                          LruArgs A) {
+  constexpr int ROW = SKC * 2 + 16, KW = 4, NC = CT * 16, TPB = CT * 256;
+  const int taps = TAPS ? TAPS : A.taps;
   __shared__ __attribute__((aligned(16))) char us[16 * ROW];
   __shared__ float red[KW][2][16][NC + 1];
   __shared__ int back[MAX_TAPS][16];     // ring row of an earlier input, or -1
@@ -361,43 +364,44 @@ __global__ __launch_bounds__(256) void lru_step_mfma(SeqView sv, LruArgs A) {
   const bf16_t* wr = (const bf16_t*)A.gw + ((u64)blk * 2 * A.n + ch) * A.n;
   const bf16_t* wi = wr + (u64)A.n * A.n;
   const s16x8 z8 = {0, 0, 0, 0, 0, 0, 0, 0};
-  for (int id = tid; id < 16 * A.taps; id += 256) {
+  for (int id = tid; id < 16 * taps; id += TPB) {
     const int i = id & 15, j = id >> 4;
     if (i < nb) {
       const int slot = sv.slots[b0 + i], p = sv.lens[slot] - j;
-      back[j][i] = p >= 0 ? slot * A.taps + p % A.taps : -1;
+      back[j][i] = p >= 0 ? slot * taps + p % taps : -1;
     }
   }
   f32x4 ar = {}, ai = {};
   for (int k0 = 0; k0 < A.n; k0 += SKC) {
     const int kn = min(SKC, A.n - k0), kp = (kn + 31) / 32 * 32;
     __syncthreads();
-    for (int id = tid; id < nb * (kp / 4); id += 256) {
+    for (int id = tid; id < nb * (kp / 4); id += TPB) {
       const int i = id / (kp / 4), k = (id % (kp / 4)) * 4;
       float v[4] = {};
       if (k < kn) {
         const int c = blk * A.n + k0 + k;
         float t[4], w[4];
         ldf4(A.cb + c, v);
-        for (int j = A.taps - 1; j > 0; --j) {
-          const int row = back[j][i];
-          if (row < 0) continue;
-          ldf4(A.ring + (u64)row * A.C + c, t);
-          ldf4(A.cw + (u64)(A.taps - 1 - j) * A.C + c, w);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = fmaf(w[e], t[e], v[e]);
+        for (int j = taps - 1; j > 0; --j) {
+          const int row = back[j][i];
+          ldf4(A.ring + (u64)max(row, 0) * A.C + c, t);
+          ldf4(A.cw + (u64)(taps - 1 - j) * A.C + c, w);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            v[e] = row < 0 ? v[e] : fmaf(w[e], t[e], v[e]);
         }
         float xb[4];
         load_x4<bf16_t>(A, b0 + i, c, t);
         ldf4(A.xb + c, xb);
-        ldf4(A.cw + (u64)(A.taps - 1) * A.C + c, w);
+        ldf4(A.cw + (u64)(taps - 1) * A.C + c, w);
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = fmaf(w[e], t[e] + xb[e], v[e]);
       }
       stf4((bf16_t*)(us + i * ROW) + k, v);
     }
     __syncthreads();
-    constexpr int U = CT == 4 ? 8 : 2;
+    constexpr int U = 2;
     for (int k = kw * 32; k < kp; k += U * KW * 32) {
       s16x8 br[U], bi[U];
 #pragma unroll
@@ -423,7 +427,7 @@ __global__ __launch_bounds__(256) void lru_step_mfma(SeqView sv, LruArgs A) {
     red[kw][1][l4 * 4 + r][ct * 16 + l15] = ai[r];
   }
   __syncthreads();
-  for (int id = tid; id < nb * NC; id += 256) {
+  for (int id = tid; id < nb * NC; id += TPB) {
     const int i = id / NC, j = id % NC;
     if (n0 + j >= A.n) continue;
     float r = A.gb[(u64)blk * 2 * A.n + n0 + j];
@@ -437,11 +441,14 @@ __global__ __launch_bounds__(256) void lru_step_mfma(SeqView sv, LruArgs A) {
     const int c = blk * A.n + n0 + j;
     const float x = ldf((const bf16_t*)A.x + (u64)row * A.ld + c) + A.xb[c];
     float u = A.cb[c];
-    for (int t = A.taps - 1; t > 0; --t)
-      if (back[t][i] >= 0)
-        u = fmaf(A.cw[(u64)(A.taps - 1 - t) * A.C + c],
-                 A.ring[(u64)back[t][i] * A.C + c], u);
-    u = fmaf(A.cw[(u64)(A.taps - 1) * A.C + c], x, u);
+#pragma unroll
+    for (int t = taps - 1; t > 0; --t) {
+      const int br = back[t][i];
+      const float v = fmaf(A.cw[(u64)(taps - 1 - t) * A.C + c],
+                           A.ring[(u64)max(br, 0) * A.C + c], u);
+      u = br < 0 ? u : v;
+    }
+    u = fmaf(A.cw[(u64)(taps - 1) * A.C + c], x, u);
     float a, z;
     lru_pair<true>(r, g, round_to(u, (const bf16_t*)nullptr),
                    A.c * softplus_f(A.lam[c]), a, z);
@@ -537,14 +544,19 @@ hipError_t lfmq_gated_lru(const SeqView& sv, const void* x, const void* y,
   if (mfma && single) {
     // wide tiles compute each convolution output less often, narrow ones
     // spread few sequences over the chip
-    if (sv.b >= 16)
-      hipLaunchKernelGGL(lru_step_mfma<4>,
-                         dim3((A.n + 63) / 64, blocks, (sv.b + 15) / 16),
-                         dim3(256), 0, stream, sv, A);
-    else
-      hipLaunchKernelGGL(lru_step_mfma<1>,
-                         dim3((A.n + 15) / 16, blocks, 1), dim3(256), 0,
-                         stream, sv, A);
+#define STEP(CT)                                                             \
+  do {                                                                       \
+    const dim3 grid((A.n + CT * 16 - 1) / (CT * 16), blocks,                 \
+                    (sv.b + 15) / 16);                                       \
+    if (taps == 4)                                                           \
+      hipLaunchKernelGGL((lru_step_mfma<CT, 4>), grid, dim3(CT * 256), 0,    \
+                         stream, sv, A);                                     \
+    else                                                                     \
+      hipLaunchKernelGGL((lru_step_mfma<CT, 0>), grid, dim3(CT * 256), 0,    \
+                         stream, sv, A);                                     \
+  } while (0)
+    if (sv.b >= 16) STEP(4); else STEP(1);
+#undef STEP
     return hipGetLastError();
   }
   const bool c4 = taps == 4 && C % 4 == 0;
